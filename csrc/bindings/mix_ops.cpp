@@ -10,6 +10,7 @@
 #include <stdint.h>
 
 #include "../kernels/mix_linrec.h"
+#include "../kernels/mix_mlstm.h"
 
 namespace rfqmix {
 void launch_embed_sinusoid(bool, const int32_t*, const int32_t*, const void*, const float*, float,
@@ -72,21 +73,32 @@ void launch_residual_add_norm(bool, float*, const void*, int64_t, bool, const vo
 bool launch_qk_norm_rotary_append(bool, const void*, int64_t, const float*, const float*,
                                   const float*, bool, int, float, const int32_t*, const float*, int,
                                   float, int, int, const int32_t*, void*, void*, int, int, int, int,
-                                  int, int, int, int, int64_t, float*, hipStream_t);
+                                  int, int, int, int, int64_t, const float*, float, float*, float*,
+                                  hipStream_t);
 bool launch_attn_keep_window(bool, const float*, const void*, const void*, int64_t, const int32_t*,
                              int, const int32_t*, const int32_t*, const int32_t*, const int32_t*,
-                             const int32_t*, int, const float*, const void*, int64_t, void*,
+                             const int32_t*, int, const float*, const void*, int64_t, int, void*,
                              int64_t, float, int, int, bool, int, int, int, int, int, hipStream_t);
 int launch_attn_keep_decode(bool, const float*, const void*, const void*, int64_t, const int32_t*,
                             int, const int32_t*, const int32_t*, const int32_t*, int, int,
-                            const float*, const void*, int64_t, void*, int64_t, float, int, int,
-                            bool, int, int, int, int, int, hipStream_t);
+                            const float*, const void*, int64_t, int, void*, int64_t, float, int,
+                            int, bool, int, int, int, int, int, hipStream_t);
 bool keep_mfma_ok(int, int, int, bool);
 bool launch_attn_keep_mfma(const float*, const void*, const void*, int64_t, const int32_t*, int,
                            const int32_t*, const int32_t*, const int32_t*, const int32_t*,
-                           const int32_t*, int, const float*, const void*, int64_t, void*, int64_t,
-                           float, int, int, bool, int, int, int, int, int, bool, int, int,
+                           const int32_t*, int, const float*, const void*, int64_t, int, void*,
+                           int64_t, float, int, int, bool, int, int, int, int, int, bool, int, int,
                            hipStream_t);
+void launch_gain_sandwich(bool, float*, const void*, int64_t, bool, const void*, int64_t, bool,
+                          const float*, int64_t, const void*, int64_t, bool, const float*, float,
+                          float, float, void*, int, int, hipStream_t);
+void launch_poly_norm_rows(bool, const void*, int64_t, void*, int64_t, int, int, float, float,
+                           float, float, float, hipStream_t);
+bool moe_route_softmax_ok(int, int);
+void launch_moe_route_softmax(const float*, int64_t, const float*, int, int, int, int, int, int,
+                              float, int32_t*, float*, float*, hipStream_t);
+bool mlstm_fuses(int, int, bool);
+bool mlstm_vec(bool, const MlstmArgs&);
 void launch_xielu_rows(bool, const void*, int64_t, void*, int64_t, int, int, float, float,
                        hipStream_t);
 void launch_rotary_append(bool, const void*, int64_t, const int32_t*, const float*, int,
@@ -652,7 +664,8 @@ void qk_norm_rotary_append(const Tensor& proj, const OptT& bias, const OptT& q_n
                            int64_t q_rot_off, int64_t k_rot_off, const Tensor& slots,
                            const OptT& k_cache, const OptT& v_cache, int64_t H, int64_t G,
                            int64_t qw, int64_t kw, int64_t vdim, int64_t v_mode,
-                           const Tensor& q_out) {
+                           const Tensor& q_out, const OptT& v_in, double v_take,
+                           const OptT& v_out) {
   const bool f32 = act_f32(proj, "qk_norm_rotary_append proj");
   TORCH_CHECK(proj.dim() == 2 && proj.stride(1) == 1, "qk_norm_rotary_append: proj [T, N]");
   const int T = (int)proj.size(0);
@@ -692,13 +705,17 @@ void qk_norm_rotary_append(const Tensor& proj, const OptT& bias, const OptT& q_n
   }
   TORCH_CHECK(q_out.dim() == 3 && q_out.size(0) == T && q_out.size(1) == H && q_out.size(2) == qw,
               "qk_norm_rotary_append: q_out [T, H, qw]");
+  TORCH_CHECK((!v_in.has_value() && !v_out.has_value()) || (v_mode != 2 && G > 0),
+              "qk_norm_rotary_append: blended values need values");
+  const int64_t nv = (int64_t)T * G * vdim;
   const float* fr = nrot > 0 ? f32p(inv_freq, "inv_freq") : nullptr;
   const bool ok = rfqmix::launch_qk_norm_rotary_append(
       f32, proj.data_ptr(), proj.stride(0), optf(bias, "bias", W), optf(q_norm_w, "q_norm_w", nqw),
       (G > 0 && k_norm_w.has_value()) ? f32p(*k_norm_w, "k_norm_w", nkw) : nullptr, norm_all,
       (int)k_norm_n, (float)eps, i32p(pos, "positions", T), fr, nrot, (float)rot_mult,
       (int)q_rot_off, (int)k_rot_off, i32p(slots, "slots", T), kp, vp, T, (int)H, (int)G, (int)qw,
-      (int)kw, (int)vdim, (int)v_mode, BS, pool_slots, const_cast<float*>(f32p(q_out, "q_out")),
+      (int)kw, (int)vdim, (int)v_mode, BS, pool_slots, optf(v_in, "v_in", nv), (float)v_take,
+      const_cast<float*>(optf(v_out, "v_out", nv)), const_cast<float*>(f32p(q_out, "q_out")),
       stream());
   TORCH_CHECK(ok, "qk_norm_rotary_append: a row does not fit the LDS");
 }
@@ -727,9 +744,12 @@ void attn_keep_window(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
   TORCH_CHECK(!sigmoid || head_bias.has_value(), "attn_keep_window: sigmoid weights need a bias");
   const void* gp = nullptr;
   int64_t gs = 0;
+  int gw = 1;                          // gate columns per head: one, or one per output
   if (gate.has_value()) {
+    gw = gate->dim() == 2 && gate->size(1) != H ? (int)vdim : 1;
     TORCH_CHECK(gate->is_cuda() && gate->scalar_type() == k_cache.scalar_type() &&
-                rows2d(*gate, T, H), "attn_keep_window: gate [T, H] in the cache's type");
+                rows2d(*gate, T, (int64_t)H * gw),
+                "attn_keep_window: gate [T, H] or [T, H vdim] in the cache's type");
     gp = gate->data_ptr();
     gs = gate->stride(0);
   }
@@ -744,7 +764,8 @@ void attn_keep_window(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
                      reinterpret_cast<uintptr_t>(q.data_ptr()) % 16 == 0 &&
                      reinterpret_cast<uintptr_t>(k_cache.data_ptr()) % 16 == 0 &&
                      reinterpret_cast<uintptr_t>(v_cache.data_ptr()) % 16 == 0 &&
-                     reinterpret_cast<uintptr_t>(out.data_ptr()) % 8 == 0;
+                     reinterpret_cast<uintptr_t>(out.data_ptr()) % 8 == 0 &&
+                     (gw == 1 || (gs % 4 == 0 && reinterpret_cast<uintptr_t>(gp) % 8 == 0));
   TORCH_CHECK(short_rows >= 0 && short_rows <= 65535 && G <= 65535, "attn_keep_window: short_rows");
   if (short_rows > 0 && !(tiles && H / G >= 16)) {
     // sequences of at most short_rows rows each (decode section): one workgroup per
@@ -753,7 +774,7 @@ void attn_keep_window(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
     const int kt = rfqmix::launch_attn_keep_decode(
         f32, f32p(q, "q"), k_cache.data_ptr(), v_cache.data_ptr(), vrs, i32p(bt, "block_tables", 0),
         (int)bt.size(1), i32p(q_start, "q_start", NB), i32p(q_len, "q_len", NB),
-        i32p(kv_len, "kv_len", NB), NB, (int)short_rows, hb, gp, gs, out.data_ptr(), out.stride(0),
+        i32p(kv_len, "kv_len", NB), NB, (int)short_rows, hb, gp, gs, gw, out.data_ptr(), out.stride(0),
         (float)scale, (int)window, (int)keep_first, sigmoid, H, G, E, (int)vdim, BS, stream());
     if (kt > 0) return;
   }
@@ -762,7 +783,7 @@ void attn_keep_window(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
         f32p(q, "q"), k_cache.data_ptr(), v_cache.data_ptr(), vrs, i32p(bt, "block_tables", 0),
         (int)bt.size(1), i32p(q_start, "q_start", NB), i32p(q_len, "q_len", NB),
         i32p(kv_len, "kv_len", NB), i32p(work_seq, "work_seq", W), i32p(work_qblk, "work_qblk", W),
-        W, hb, gp, gs, out.data_ptr(), out.stride(0), (float)scale, (int)window, (int)keep_first,
+        W, hb, gp, gs, gw, out.data_ptr(), out.stride(0), (float)scale, (int)window, (int)keep_first,
         sigmoid, H, G, E, (int)vdim, BS, shared, NB, (int)short_rows, stream());
     return;
   }
@@ -770,7 +791,7 @@ void attn_keep_window(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
       f32, f32p(q, "q"), k_cache.data_ptr(), v_cache.data_ptr(), vrs, i32p(bt, "block_tables", 0),
       (int)bt.size(1), i32p(q_start, "q_start", NB), i32p(q_len, "q_len", NB),
       i32p(kv_len, "kv_len", NB), i32p(work_seq, "work_seq", W), i32p(work_qblk, "work_qblk", W), W,
-      hb, gp, gs, out.data_ptr(), out.stride(0), (float)scale, (int)window, (int)keep_first,
+      hb, gp, gs, gw, out.data_ptr(), out.stride(0), (float)scale, (int)window, (int)keep_first,
       sigmoid, H, G, E, (int)vdim, BS, stream());
   TORCH_CHECK(ok, "attn_keep_window: value size too large for the LDS");
 }
@@ -900,9 +921,141 @@ void gelu_rows(const Tensor& x, const Tensor& out) {
                            (int)x.size(0), (int)x.size(1), stream());
 }
 
+void gain_sandwich(const Tensor& x, const OptT& y, const OptT& y2, const OptT& y2_logit,
+                   const OptT& h_in, const OptT& h_weight, double g_post, double g_pre, double eps,
+                   const OptT& out) {
+  TORCH_CHECK(x.dim() == 2 && x.size(1) >= 1, "gain_sandwich: x [T, d]");
+  const int T = (int)x.size(0), d = (int)x.size(1);
+  const void* p[3] = {nullptr, nullptr, nullptr};
+  int64_t st[3] = {0, 0, 0};
+  bool f[3] = {true, true, true};
+  const OptT* in[3] = {&y, &y2, &h_in};
+  for (int i = 0; i < 3; ++i)
+    if (in[i]->has_value()) {
+      const Tensor& u = **in[i];
+      f[i] = act_f32(u, "gain_sandwich input");
+      TORCH_CHECK(rows2d(u, T, d), "gain_sandwich: y, y2, h_in [T, d]");
+      p[i] = u.data_ptr();
+      st[i] = u.stride(0);
+    }
+  const float* lp = nullptr;
+  int64_t ls = 0;
+  if (y2.has_value()) {
+    TORCH_CHECK(y2_logit.has_value() && y2_logit->is_cuda() &&
+                y2_logit->scalar_type() == at::kFloat && y2_logit->dim() == 1 &&
+                y2_logit->size(0) == T, "gain_sandwich: y2_logit [T] float32");
+    lp = y2_logit->data_ptr<float>();
+    ls = y2_logit->stride(0);
+  }
+  TORCH_CHECK(!h_in.has_value() || h_weight.has_value(), "gain_sandwich: h_in needs h_weight");
+  bool of32 = true;
+  void* op = nullptr;
+  if (out.has_value()) {
+    of32 = act_f32(*out, "gain_sandwich out");
+    TORCH_CHECK(rows2d(*out, T, d) && out->is_contiguous(), "gain_sandwich: out [T, d]");
+    op = out->data_ptr();
+  }
+  rfqmix::launch_gain_sandwich(of32, const_cast<float*>(f32p(x, "x")), p[0], st[0], f[0], p[1],
+                               st[1], f[1], lp, ls, p[2], st[2], f[2],
+                               h_in.has_value() ? f32p(*h_weight, "h_weight", T) : nullptr,
+                               (float)g_post, (float)g_pre, (float)eps, op, T, d, stream());
+}
+
+void poly_norm_rows(const Tensor& x, double a, double b, double c, double e, double eps,
+                    const Tensor& out) {
+  const bool f32 = act_f32(x, "poly_norm_rows x");
+  TORCH_CHECK(x.dim() == 2 && x.stride(1) == 1 && out.is_cuda() &&
+              out.scalar_type() == x.scalar_type() && rows2d(out, x.size(0), x.size(1)),
+              "poly_norm_rows: x, out [T, F] of one type");
+  rfqmix::launch_poly_norm_rows(f32, x.data_ptr(), x.stride(0), out.data_ptr(), out.stride(0),
+                                (int)x.size(0), (int)x.size(1), (float)a, (float)b, (float)c,
+                                (float)e, (float)eps, stream());
+}
+
+void moe_route_softmax(const Tensor& z, const Tensor& corr, int64_t real, int64_t top,
+                       int64_t groups, int64_t keep, double scale, const Tensor& ids,
+                       const Tensor& weights, const OptT& ident) {
+  TORCH_CHECK(z.dim() == 2 && z.stride(1) == 1 && z.is_cuda() && z.scalar_type() == at::kFloat,
+              "moe_route_softmax: z [T, >= n] float32");
+  const int T = (int)z.size(0), E = (int)corr.numel();
+  TORCH_CHECK(z.size(1) >= E && real >= 1 && real <= E && top >= 1 && top <= E,
+              "moe_route_softmax: sizes");
+  TORCH_CHECK(groups == 0 || (E % groups == 0 && keep >= 1 && keep <= groups &&
+                              top <= keep * (E / groups)), "moe_route_softmax: groups");
+  TORCH_CHECK(rfqmix::moe_route_softmax_ok(E, (int)groups), "moe_route_softmax: too many experts");
+  TORCH_CHECK(ident.has_value() || real == E, "moe_route_softmax: identity experts need ident");
+  TORCH_CHECK(ids.is_cuda() && ids.scalar_type() == at::kInt && ids.is_contiguous() &&
+              ids.numel() == (int64_t)T * top, "moe_route_softmax: ids [T, top] int32");
+  rfqmix::launch_moe_route_softmax(
+      z.data_ptr<float>(), z.stride(0), f32p(corr, "correction", E), T, E, (int)real, (int)top,
+      (int)groups, (int)keep, (float)scale, ids.data_ptr<int32_t>(),
+      const_cast<float*>(f32p(weights, "weights", (int64_t)T * top)),
+      const_cast<float*>(optf(ident, "ident", T)), stream());
+}
+
+void mlstm_recurrence(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& z,
+                      const Tensor& zbias, double cap, double q_scale, const Tensor& gate,
+                      const Tensor& norm_w, double eps, const Tensor& S, const Tensor& n,
+                      const Tensor& m, const Tensor& row_state, const Tensor& row_back,
+                      const Tensor& row_fwd, const Tensor& pos, const OptT& run_rows,
+                      const Tensor& out, const OptT& raw, bool chunked) {
+  const bool f32 = act_f32(out, "mlstm_recurrence out");
+  TORCH_CHECK(S.dim() == 4 && S.size(0) % 2 == 0, "mlstm_recurrence: S [2 slots, H, dim, vdim]");
+  const int H = (int)S.size(1), dim = (int)S.size(2), vdim = (int)S.size(3);
+  TORCH_CHECK(out.dim() == 2, "mlstm_recurrence: out [T, H vdim]");
+  const int T = (int)out.size(0);
+  const Tensor* in[4] = {&q, &k, &v, &gate};
+  const int64_t w[4] = {(int64_t)H * dim, (int64_t)H * dim, (int64_t)H * vdim, (int64_t)H * vdim};
+  for (int i = 0; i < 4; ++i)
+    TORCH_CHECK(in[i]->is_cuda() && in[i]->scalar_type() == out.scalar_type() &&
+                rows2d(*in[i], T, w[i]), "mlstm_recurrence: q, k [T, H dim], v, gate [T, H vdim]");
+  TORCH_CHECK(z.is_cuda() && z.scalar_type() == at::kFloat && rows2d(z, T, 2 * (int64_t)H),
+              "mlstm_recurrence: z [T, 2 H] float32");
+  TORCH_CHECK(rows2d(out, T, (int64_t)H * vdim) && out.is_contiguous(),
+              "mlstm_recurrence: out [T, H vdim]");
+  TORCH_CHECK(rfqmix::mlstm_ok(dim, vdim) && H <= 65535 && cap > 0,
+              "mlstm_recurrence: sizes outside the kernel's range");
+  rfqmix::MlstmArgs a;
+  a.q = q.data_ptr(); a.k = k.data_ptr(); a.v = v.data_ptr();
+  a.qs = q.stride(0); a.ks = k.stride(0); a.vs = v.stride(0);
+  a.z = z.data_ptr<float>(); a.zs = z.stride(0);
+  a.zbias = f32p(zbias, "zbias", 2 * (int64_t)H);
+  a.cap = (float)cap; a.q_scale = (float)q_scale;
+  a.gate = gate.data_ptr(); a.gs = gate.stride(0);
+  a.norm_w = f32p(norm_w, "norm_w", (int64_t)H * vdim);
+  a.eps = (float)eps;
+  a.raw = raw.has_value() ? const_cast<float*>(f32p(*raw, "raw", (int64_t)T * H * vdim)) : nullptr;
+  a.S = const_cast<float*>(f32p(S, "S"));
+  a.n = const_cast<float*>(f32p(n, "n", S.size(0) * H * dim));
+  a.m = const_cast<float*>(f32p(m, "m", S.size(0) * H));
+  a.row_state = i32p(row_state, "row_state", T); a.row_back = i32p(row_back, "row_back", T);
+  a.row_fwd = i32p(row_fwd, "row_fwd", T); a.pos = i32p(pos, "positions", T);
+  a.run_rows = run_rows.has_value() ? i32p(*run_rows, "run_rows", 0) : nullptr;
+  a.runs = run_rows.has_value() ? (int)run_rows->numel() : 0;
+  a.out = out.data_ptr();
+  a.T = T; a.H = H; a.dim = dim; a.vdim = vdim; a.slots = (int)S.size(0) / 2;
+  TORCH_CHECK(raw.has_value() || rfqmix::mlstm_fuses(dim, vdim, rfqmix::mlstm_vec(f32, a)),
+              "mlstm_recurrence: a head of this size needs raw");
+  if (chunked && !f32 && raw.has_value() && rfqmix::launch_mlstm_chunk(a, stream())) return;
+  rfqmix::launch_mlstm(f32, a, stream());
+}
+
+bool mlstm_fused_ok(int64_t dim, int64_t vdim) {
+  return rfqmix::mlstm_fuses((int)dim, (int)vdim, true) && rfqmix::mlstm_fuses((int)dim, (int)vdim, false);
+}
+bool mlstm_chunk_ok(int64_t dim, int64_t vdim) {
+  return rfqmix::mlstm_chunk_ok((int)dim, (int)vdim);
+}
+
 }  // namespace
 
 TORCH_LIBRARY(rfq_mix, m) {
+  m.def("gain_sandwich(Tensor(a!) x, Tensor? y, Tensor? y2, Tensor? y2_logit, Tensor? h_in, Tensor? h_weight, float g_post, float g_pre, float eps, Tensor(b!)? out) -> ()");
+  m.def("poly_norm_rows(Tensor x, float a, float b, float c, float e, float eps, Tensor(a!) out) -> ()");
+  m.def("moe_route_softmax(Tensor z, Tensor correction, int real, int top, int groups, int keep, float scale, Tensor(a!) ids, Tensor(b!) weights, Tensor(c!)? ident) -> ()");
+  m.def("mlstm_recurrence(Tensor q, Tensor k, Tensor v, Tensor z, Tensor zbias, float cap, float q_scale, Tensor gate, Tensor norm_w, float eps, Tensor(a!) S, Tensor(b!) n, Tensor(c!) m, Tensor row_state, Tensor row_back, Tensor row_fwd, Tensor pos, Tensor? run_rows, Tensor(d!) out, Tensor(e!)? raw, bool chunked) -> ()");
+  m.def("mlstm_fused_ok", &mlstm_fused_ok);
+  m.def("mlstm_chunk_ok", &mlstm_chunk_ok);
   m.def("embed_sinusoid(Tensor ids, Tensor pos, Tensor table, Tensor inv_freq, float scale, Tensor(a!) out) -> ()");
   m.def("sandwich_norm(Tensor? y, Tensor(a!) residual, Tensor? w_post, Tensor? gain, Tensor w_pre, float eps, Tensor(b!) out) -> ()");
   m.def("canon_conv(Tensor h, Tensor w, Tensor(a!) state, Tensor row_state, Tensor row_back, Tensor row_fwd, Tensor pos, Tensor(b!) out) -> ()");
@@ -928,7 +1081,7 @@ TORCH_LIBRARY(rfq_mix, m) {
   m.def("rotary_append(Tensor qkv, Tensor pos, Tensor inv_freq, Tensor slots, Tensor(a!) k_cache, Tensor(b!) v_cache, int H, int G, int maps, int dim, int vdim, Tensor(c!) q_out) -> ()");
   m.def("attn_diff_window(Tensor q, Tensor k_cache, Tensor v_cache, Tensor bt, Tensor q_start, Tensor q_len, Tensor kv_len, Tensor work_seq, Tensor work_qblk, Tensor gate, Tensor(a!) out, float scale, int window, float lam, float eps, float out_mult, int short_rows, bool mfma) -> ()");
   m.def("diff_mfma_ok", &diff_mfma_ok);
-  m.def("qk_norm_rotary_append(Tensor proj, Tensor? bias, Tensor? q_norm_w, Tensor? k_norm_w, bool norm_all, int k_norm_n, float eps, Tensor pos, Tensor inv_freq, float rot_mult, int q_rot_off, int k_rot_off, Tensor slots, Tensor(a!)? k_cache, Tensor(b!)? v_cache, int H, int G, int qw, int kw, int vdim, int v_mode, Tensor(c!) q_out) -> ()");
+  m.def("qk_norm_rotary_append(Tensor proj, Tensor? bias, Tensor? q_norm_w, Tensor? k_norm_w, bool norm_all, int k_norm_n, float eps, Tensor pos, Tensor inv_freq, float rot_mult, int q_rot_off, int k_rot_off, Tensor slots, Tensor(a!)? k_cache, Tensor(b!)? v_cache, int H, int G, int qw, int kw, int vdim, int v_mode, Tensor(c!) q_out, Tensor? v_in, float v_take, Tensor(d!)? v_out) -> ()");
   m.def("attn_keep_window(Tensor q, Tensor k_cache, Tensor v_cache, int vdim, Tensor bt, Tensor q_start, Tensor q_len, Tensor kv_len, Tensor work_seq, Tensor work_qblk, Tensor? head_bias, Tensor? gate, Tensor(a!) out, float scale, int window, int keep_first, bool sigmoid, int short_rows, bool mfma) -> ()");
   m.def("keep_mfma_ok", &keep_mfma_ok);
   m.def("xielu_rows(Tensor x, float ap, float an, Tensor(a!) out) -> ()");
@@ -941,6 +1094,10 @@ TORCH_LIBRARY(rfq_mix, m) {
 }
 
 TORCH_LIBRARY_IMPL(rfq_mix, CUDA, m) {
+  m.impl("gain_sandwich", &gain_sandwich);
+  m.impl("poly_norm_rows", &poly_norm_rows);
+  m.impl("moe_route_softmax", &moe_route_softmax);
+  m.impl("mlstm_recurrence", &mlstm_recurrence);
   m.impl("embed_sinusoid", &embed_sinusoid);
   m.impl("sandwich_norm", &sandwich_norm);
   m.impl("canon_conv", &canon_conv);

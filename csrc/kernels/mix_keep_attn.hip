@@ -4,12 +4,15 @@
 //   qk_norm_rotary_append   rows q [H, qw] | k [G, kw] (| v [G, vdim]) of a fused projection:
 //                           bias, RMS norm per head or over the whole projection, rotation of
 //                           entries (off + i, off + i + n) by pos * f_i with a factor on cos and
-//                           sin; q out in fp32, k and the values into their page rows
+//                           sin; q out in fp32, k and the values into their page rows; the
+//                           values may be blended with another layer's values of the same token
+//                           (v <- keep v + take v_in) and handed on unblended (v_out)
 //   attn_keep_window        s(i, j) = scale q_h(i) . k_g(j);  i sees j <= i with
 //                           i - j < window or j < keep_first (window 0: every j <= i)
 //                             softmax:  w = exp(s) / (sum_j' exp(s(i, j')) [+ exp(bias_h)])
 //                             sigmoid:  w = 1 / (1 + exp(-(s + bias_h))), not normalised
-//                           out(i) = sum_j w v_g(j) [* sigmoid(gate(i, h))]
+//                           out(i) = sum_j w v_g(j) [* sigmoid(gate(i, h)) or, with a gate column
+//                           per output (gate_w = vdim), * sigmoid(gate(i, h, dv))]
 //                           The values are the first vdim entries of rows of stride vrs, so the
 //                           key pages themselves can be the values (latent attention).
 //   xielu_rows              z > 0: ap z^2 + z / 2;  z <= 0: an (exp(z) - 1 - z) + z / 2
@@ -92,7 +95,8 @@ __global__ __launch_bounds__(256) void qk_norm_rotary_append_kernel(
     int k_norm_n, float eps, const int32_t* __restrict__ pos, const float* __restrict__ inv_freq,
     int nrot, float rot_mult, int q_rot_off, int k_rot_off, const int32_t* __restrict__ slots,
     T* __restrict__ k_cache, T* __restrict__ v_cache, int H, int G, int qw, int kw, int vdim,
-    int v_mode, int BS, int64_t pool_slots, float* __restrict__ q_out) {
+    int v_mode, int BS, int64_t pool_slots, const float* __restrict__ v_in, float v_keep,
+    float v_take, float* __restrict__ v_out, float* __restrict__ q_out) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int t = blockIdx.x, tid = threadIdx.x, nthr = blockDim.x;
   const int lane = tid & 63, wid = tid >> 6, nw = nthr >> 6;
@@ -175,8 +179,23 @@ __global__ __launch_bounds__(256) void qk_norm_rotary_append_kernel(
     const float* vs = v_mode == 0 ? row + nq + nk : row + nq;
     for (int x = tid * CW; x < G * vdim; x += nthr * CW) {
       const int g = x / vdim, e = x - g * vdim;
-      st_chunk<CW>(v_cache + (page_row + (int64_t)g * BS) * vdim + e, vs + x);
+      T* dst = v_cache + (page_row + (int64_t)g * BS) * vdim + e;
+      if (v_in == nullptr) {
+        st_chunk<CW>(dst, vs + x);
+        continue;
+      }
+      float f[CW], u[CW];
+      ld_chunk<CW>(vs + x, f);
+      ld_chunk<CW>(v_in + (int64_t)t * G * vdim + x, u);
+#pragma unroll
+      for (int i = 0; i < CW; ++i) f[i] = v_keep * f[i] + v_take * u[i];
+      st_chunk<CW>(dst, f);
     }
+  }
+  if (v_out != nullptr) {               // as projected, for the layers that blend them in
+    const float* vs = v_mode == 0 ? row + nq + nk : row + nq;
+    for (int x = tid * CW; x < G * vdim; x += nthr * CW)
+      st_chunk<CW>(v_out + (int64_t)t * G * vdim + x, vs + x);
   }
   // q and k: norm factor and weight, then the rotation (the partner entry is normed on the way).
   // CW = 8: the normed width, the rotation's offset and its half are multiples of 8, so a chunk
@@ -256,7 +275,8 @@ __global__ __launch_bounds__(256) void attn_keep_window_kernel(
     const int32_t* __restrict__ q_start, const int32_t* __restrict__ q_len,
     const int32_t* __restrict__ kv_len, const int32_t* __restrict__ work_seq,
     const int32_t* __restrict__ work_qblk, const float* __restrict__ head_bias,
-    const T* __restrict__ gate, int64_t gate_stride, T* __restrict__ out, int64_t out_stride,
+    const T* __restrict__ gate, int64_t gate_stride, int gate_w, T* __restrict__ out,
+    int64_t out_stride,
     float scale, int window, int keep_first, int sigmoid, int H, int G, int E, int vdim, int BS) {
   const int s = work_seq[blockIdx.x];
   if (s < 0) return;
@@ -384,7 +404,8 @@ __global__ __launch_bounds__(256) void attn_keep_window_kernel(
     const int i = x / vdim, dv = x - i * vdim;
     const int64_t t = q_start[s] + i0 + i;
     float mul = sigmoid ? 1.f : (ll[i] > 0.f ? 1.0f / ll[i] : 0.f);
-    if (gate != nullptr) mul /= 1.0f + expf(-ldf(gate + t * gate_stride + hh));
+    if (gate != nullptr)
+      mul /= 1.0f + expf(-ldf(gate + t * gate_stride + (gate_w == 1 ? hh : hh * vdim + dv)));
     stf(out + t * out_stride + (int64_t)hh * vdim + dv, Os[x] * mul);
   }
 }
@@ -402,7 +423,8 @@ __global__ __launch_bounds__(256) void attn_keep_decode_kernel(
     int64_t vrs, const int32_t* __restrict__ block_tables, int maxb,
     const int32_t* __restrict__ q_start, const int32_t* __restrict__ q_len,
     const int32_t* __restrict__ kv_len, const float* __restrict__ head_bias,
-    const T* __restrict__ gate, int64_t gate_stride, T* __restrict__ out, int64_t out_stride,
+    const T* __restrict__ gate, int64_t gate_stride, int gate_w, T* __restrict__ out,
+    int64_t out_stride,
     float scale, int window, int keep_first, int sigmoid, int H, int G, int E, int vdim, int BS,
     int KT) {
   const int s = blockIdx.x, g = blockIdx.y;
@@ -581,9 +603,13 @@ __global__ __launch_bounds__(256) void attn_keep_decode_kernel(
     for (int hr = wid; hr < R; hr += nw) {
       const int hh = g * R + hr;
       float mul = sigmoid ? 1.f : (lrow[hr] > 0.f ? 1.0f / lrow[hr] : 0.f);
-      if (gate != nullptr) mul /= 1.0f + expf(-ldf(gate + (int64_t)t * gate_stride + hh));
-      for (int dv = lane; dv < vdim; dv += 64)
-        stf(out + (int64_t)t * out_stride + (int64_t)hh * vdim + dv, acc[hr * vdim + dv] * mul);
+      const T* gr = gate == nullptr ? nullptr : gate + (int64_t)t * gate_stride;
+      if (gr != nullptr && gate_w == 1) mul /= 1.0f + expf(-ldf(gr + hh));
+      for (int dv = lane; dv < vdim; dv += 64) {
+        float o = acc[hr * vdim + dv] * mul;
+        if (gr != nullptr && gate_w > 1) o /= 1.0f + expf(-ldf(gr + hh * vdim + dv));
+        stf(out + (int64_t)t * out_stride + (int64_t)hh * vdim + dv, o);
+      }
     }
   }
 }
@@ -620,7 +646,8 @@ bool launch_qk_norm_rotary_append(bool f32, const void* proj, int64_t stride, co
                                   const float* inv_freq, int nrot, float rot_mult, int q_rot_off,
                                   int k_rot_off, const int32_t* slots, void* k_cache, void* v_cache,
                                   int T, int H, int G, int qw, int kw, int vdim, int v_mode, int BS,
-                                  int64_t pool_slots, float* q_out, hipStream_t s) {
+                                  int64_t pool_slots, const float* v_in, float v_take,
+                                  float* v_out, float* q_out, hipStream_t s) {
   const size_t W = (size_t)H * qw + (size_t)G * kw + (v_mode == 0 ? (size_t)G * vdim : 0);
   const size_t lds = (W + 4 + H + G + 4 + 2 * (size_t)nrot + 16) * sizeof(float);
   if (lds > (size_t)kLdsMax) return false;
@@ -637,12 +664,14 @@ bool launch_qk_norm_rotary_append(bool f32, const void* proj, int64_t stride, co
   const bool vec = qw % 8 == 0 && (G == 0 || kw % 8 == 0) && (v_mode == 2 || vdim % 8 == 0) &&
                    stride % 8 == 0 && k_norm_n % 8 == 0 && nrot % 8 == 0 && q_rot_off % 8 == 0 &&
                    k_rot_off % 8 == 0 && al16(proj) && al16(bias) && al16(q_norm_w) &&
-                   al16(k_norm_w) && al16(k_cache) && al16(v_cache) && al16(q_out);
+                   al16(k_norm_w) && al16(k_cache) && al16(v_cache) && al16(q_out) && al16(v_in) &&
+                   al16(v_out);
 #define QKN_GO(TT, CW)                                                                          \
   hipLaunchKernelGGL((qk_norm_rotary_append_kernel<TT, CW>), dim3(T), dim3(256), lds, s,       \
                      (const TT*)proj, stride, bias, q_norm_w, k_norm_w, (int)norm_all, k_norm_n, \
                      eps, pos, inv_freq, nrot, rot_mult, q_rot_off, k_rot_off, slots,           \
-                     (TT*)k_cache, (TT*)v_cache, H, G, qw, kw, vdim, v_mode, BS, pool_slots, q_out)
+                     (TT*)k_cache, (TT*)v_cache, H, G, qw, kw, vdim, v_mode, BS, pool_slots,    \
+                     v_in, 1.0f - v_take, v_take, v_out, q_out)
   if (f32) {
     if (vec) QKN_GO(float, 8);
     else QKN_GO(float, 1);
@@ -658,8 +687,8 @@ bool launch_attn_keep_window(bool f32, const float* q, const void* k_cache, cons
                              int64_t vrs, const int32_t* bt, int maxb, const int32_t* q_start,
                              const int32_t* q_len, const int32_t* kv_len, const int32_t* work_seq,
                              const int32_t* work_qblk, int W, const float* head_bias,
-                             const void* gate, int64_t gate_stride, void* out, int64_t out_stride,
-                             float scale, int window, int keep_first, bool sigmoid, int H, int G,
+                             const void* gate, int64_t gate_stride, int gate_w, void* out,
+                             int64_t out_stride, float scale, int window, int keep_first, bool sigmoid, int H, int G,
                              int E, int vdim, int BS, hipStream_t s) {
   const size_t lds = ((size_t)KQB * (KEC + 1) + (size_t)KKT * (KEC + 1) + (size_t)KQB * (KKT + 1) +
                       (size_t)KQB * vdim + 2 * KQB) * sizeof(float);
@@ -674,13 +703,13 @@ bool launch_attn_keep_window(bool f32, const float* q, const void* k_cache, cons
   if (f32)
     hipLaunchKernelGGL(attn_keep_window_kernel<float>, dim3(W, H), dim3(256), lds, s, q,
                        (const float*)k_cache, (const float*)v_cache, vrs, bt, maxb, q_start, q_len,
-                       kv_len, work_seq, work_qblk, head_bias, (const float*)gate, gate_stride,
+                       kv_len, work_seq, work_qblk, head_bias, (const float*)gate, gate_stride, gate_w,
                        (float*)out, out_stride, scale, window, keep_first, (int)sigmoid, H, G, E,
                        vdim, BS);
   else
     hipLaunchKernelGGL(attn_keep_window_kernel<bf16_t>, dim3(W, H), dim3(256), lds, s, q,
                        (const bf16_t*)k_cache, (const bf16_t*)v_cache, vrs, bt, maxb, q_start, q_len,
-                       kv_len, work_seq, work_qblk, head_bias, (const bf16_t*)gate, gate_stride,
+                       kv_len, work_seq, work_qblk, head_bias, (const bf16_t*)gate, gate_stride, gate_w,
                        (bf16_t*)out, out_stride, scale, window, keep_first, (int)sigmoid, H, G, E,
                        vdim, BS);
   return true;
@@ -696,8 +725,8 @@ static size_t attn_keep_decode_floats(int R, int E, int vdim, int KT) {
 int launch_attn_keep_decode(bool f32, const float* q, const void* k_cache, const void* v_cache,
                             int64_t vrs, const int32_t* bt, int maxb, const int32_t* q_start,
                             const int32_t* q_len, const int32_t* kv_len, int NA, int max_rows,
-                            const float* head_bias, const void* gate, int64_t gate_stride, void* out,
-                            int64_t out_stride, float scale, int window, int keep_first,
+                            const float* head_bias, const void* gate, int64_t gate_stride,
+                            int gate_w, void* out, int64_t out_stride, float scale, int window, int keep_first,
                             bool sigmoid, int H, int G, int E, int vdim, int BS, hipStream_t s) {
   const int R = H / G;
   int KT = 64;
@@ -719,12 +748,12 @@ int launch_attn_keep_decode(bool f32, const float* q, const void* k_cache, const
   if (f32)
     hipLaunchKernelGGL(attn_keep_decode_kernel<float>, grid, dim3(256), lds, s, q,
                        (const float*)k_cache, (const float*)v_cache, vrs, bt, maxb, q_start, q_len,
-                       kv_len, head_bias, (const float*)gate, gate_stride, (float*)out, out_stride,
+                       kv_len, head_bias, (const float*)gate, gate_stride, gate_w, (float*)out, out_stride,
                        scale, window, keep_first, (int)sigmoid, H, G, E, vdim, BS, KT);
   else
     hipLaunchKernelGGL(attn_keep_decode_kernel<bf16_t>, grid, dim3(256), lds, s, q,
                        (const bf16_t*)k_cache, (const bf16_t*)v_cache, vrs, bt, maxb, q_start, q_len,
-                       kv_len, head_bias, (const bf16_t*)gate, gate_stride, (bf16_t*)out, out_stride,
+                       kv_len, head_bias, (const bf16_t*)gate, gate_stride, gate_w, (bf16_t*)out, out_stride,
                        scale, window, keep_first, (int)sigmoid, H, G, E, vdim, BS, KT);
   return KT;
 }

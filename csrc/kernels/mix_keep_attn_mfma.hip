@@ -1,6 +1,7 @@
 // attn_keep_window on MFMA tiles (bf16 pages of 32 tokens, key width a multiple of 32, value
 // width a multiple of 16).  Semantics of mix_keep_attn.hip: sliding window with kept first
-// tokens; softmax, softmax with a sink, or unnormalised sigmoid weights; optional output gate;
+// tokens; softmax, softmax with a sink, or unnormalised sigmoid weights; optional output gate
+// (a column per head, or gate_w = vdim: one per output, rows 8-byte aligned);
 // the values may be the leading entries of the key rows themselves (latent attention).
 //
 // One workgroup per (work item, HPW heads of one key/value head); a work item is (sequence,
@@ -57,8 +58,8 @@ __global__ __launch_bounds__(128 * HPW) void attn_keep_mfma_kernel(
     int maxb, const int32_t* __restrict__ q_start, const int32_t* __restrict__ q_len,
     const int32_t* __restrict__ kv_len, const int32_t* __restrict__ work_seq,
     const int32_t* __restrict__ work_qblk, const float* __restrict__ head_bias,
-    const bf16_t* __restrict__ gate, int64_t gate_stride, bf16_t* __restrict__ out,
-    int64_t out_stride, float scale, int window, int keep_first, int sigmoid, int H, int G) {
+    const bf16_t* __restrict__ gate, int64_t gate_stride, int gate_w,
+    bf16_t* __restrict__ out, int64_t out_stride, float scale, int window, int keep_first, int sigmoid, int H, int G) {
   constexpr int E = 32 * DK, vdim = 16 * DV, NT = 128 * HPW;
   constexpr int KRS = E + 8;                       // shorts per key row in LDS (+ 16 bytes)
   constexpr int VRS = SHARED ? KRS : vdim + 8;     // shorts per value row
@@ -256,10 +257,20 @@ __global__ __launch_bounds__(128 * HPW) void attn_keep_mfma_kernel(
   // lane (col, grp) holds value channels 16 m + 4 grp .. + 3 of its column: 8-byte stores
   if (qlive) {
     float mul = sigmoid ? 1.f : (lrun > 0.f ? 1.0f / lrun : 0.f);
-    if (gate != nullptr) mul /= 1.0f + __expf(-ldf(gate + t * gate_stride + hh));
+    if (gate != nullptr && gate_w == 1) mul /= 1.0f + __expf(-ldf(gate + t * gate_stride + hh));
+    // a gate column per output: four neighbouring logits per 16-channel block, 8-byte reads
+    const bf16_t* grow = gate != nullptr && gate_w > 1
+                             ? gate + t * gate_stride + (int64_t)hh * vdim + grp * 4 : nullptr;
     bf16_t* orow = out + t * out_stride + (int64_t)hh * vdim + grp * 4;
 #pragma unroll
     for (int m = 0; m < DV; ++m) {
+      if (grow != nullptr) {
+        const uint2 gu = *reinterpret_cast<const uint2*>(grow + m * 16);
+        o[m][0] /= 1.0f + __expf(-__uint_as_float(gu.x << 16));
+        o[m][1] /= 1.0f + __expf(-__uint_as_float(gu.x & 0xffff0000u));
+        o[m][2] /= 1.0f + __expf(-__uint_as_float(gu.y << 16));
+        o[m][3] /= 1.0f + __expf(-__uint_as_float(gu.y & 0xffff0000u));
+      }
       bf16_t b[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i) stf(&b[i], o[m][i] * mul);
@@ -295,6 +306,7 @@ struct KeepArgs {
   const float* head_bias;
   const void* gate;
   int64_t gate_stride;
+  int gate_w;
   void* out;
   int64_t out_stride;
   float scale;
@@ -325,7 +337,7 @@ static void launch_keep_mfma_one(const KeepArgs& a) {
                      dim3(128 * HPW), lds, a.s, a.q, (const bf16_t*)a.k_cache,
                      (const bf16_t*)a.v_cache, a.vrs, a.bt, a.maxb, a.q_start, a.q_len, a.kv_len,
                      a.work_seq, a.work_qblk, a.head_bias, (const bf16_t*)a.gate, a.gate_stride,
-                     (bf16_t*)a.out, a.out_stride, a.scale, a.window, a.keep_first, (int)a.sigmoid,
+                     a.gate_w, (bf16_t*)a.out, a.out_stride, a.scale, a.window, a.keep_first, (int)a.sigmoid,
                      a.H, a.G);
 }
 
@@ -340,14 +352,14 @@ bool launch_attn_keep_mfma(const float* q, const void* k_cache, const void* v_ca
                            const int32_t* bt, int maxb, const int32_t* q_start,
                            const int32_t* q_len, const int32_t* kv_len, const int32_t* work_seq,
                            const int32_t* work_qblk, int W, const float* head_bias,
-                           const void* gate, int64_t gate_stride, void* out, int64_t out_stride,
-                           float scale, int window, int keep_first, bool sigmoid, int H, int G,
+                           const void* gate, int64_t gate_stride, int gate_w, void* out,
+                           int64_t out_stride, float scale, int window, int keep_first, bool sigmoid, int H, int G,
                            int E, int vdim, int BS, bool shared, int NA, int short_rows,
                            hipStream_t s) {
   if (!keep_mfma_ok(E, vdim, BS, shared)) return false;
   if (short_rows > 0 ? NA == 0 : W == 0) return true;
   const KeepArgs a{q, k_cache, v_cache, vrs, bt, maxb, q_start, q_len, kv_len, work_seq, work_qblk,
-                   W, head_bias, gate, gate_stride, out, out_stride, scale, window, keep_first,
+                   W, head_bias, gate, gate_stride, gate_w, out, out_stride, scale, window, keep_first,
                    sigmoid, H, G, NA, short_rows, s};
   const int DK = E / 32, DV = vdim / 16;
   if (shared) {

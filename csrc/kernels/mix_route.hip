@@ -1,4 +1,5 @@
-// Mixture of experts with grouped sigmoid routing, any sizes, either activation type.
+// Mixture of experts with grouped sigmoid routing or grouped softmax routing with identity
+// experts, any sizes, either activation type.  Sigmoid routing:
 //
 //   s = sigmoid(z)                       router scores (z: fp32 router logits)
 //   choice = s + correction              chooses; the weights use s
@@ -64,6 +65,108 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(
   }
   const float inv = 1.0f / (sum + 1e-20f);
   for (int a = 0; a < top; ++a) wt[a] *= inv;
+}
+
+// Softmax routing over `real` experts followed by identity experts (whose output is their input),
+// n = E columns of z in all:
+//   s = softmax(z);  choice = s + correction (chooses; the weights use s)
+//   a group's score is its largest choice score; only the `keep` best of `groups` equal groups of
+//   neighbours can be chosen (groups 0: no limit)
+//   weights = scale * s[chosen], not renormalised
+// A chosen identity expert is written as id `real` with weight 0 (a segment no expert kernel
+// computes) and its weight is added to ident[t].  One wave per token: a lane holds columns lane,
+// lane + 64, ...; ties go to the lower index.  LDS: choice[E] | s[E] | group[groups].
+__global__ __launch_bounds__(64) void moe_route_softmax_kernel(
+    const float* __restrict__ z, int64_t zs, const float* __restrict__ corr, int E, int real,
+    int top, int groups, int keep, float scale, int32_t* __restrict__ ids,
+    float* __restrict__ weights, float* __restrict__ ident) {
+  extern __shared__ float lds[];
+  float* ch = lds;
+  float* sc = ch + E;
+  float* gr = sc + E;
+  const int t = blockIdx.x, lane = threadIdx.x;
+  const float* zr = z + (int64_t)t * zs;
+  float mx = kNegInfR;
+  for (int e = lane; e < E; e += 64) mx = fmaxf(mx, zr[e]);
+  mx = wave_max(mx);
+  float sum = 0.f;
+  for (int e = lane; e < E; e += 64) {
+    const float p = expf(zr[e] - mx);
+    sc[e] = p;
+    sum += p;
+  }
+  const float inv = 1.0f / wave_sum(sum);
+  for (int e = lane; e < E; e += 64) {
+    const float p = sc[e] * inv;
+    sc[e] = p;
+    ch[e] = p + corr[e];
+  }
+  __syncthreads();
+  // the largest of v[0 .. n) in every lane (index n: nothing left); taken ones are -inf
+  auto best_of = [&](const float* v, int n) {
+    float b = kNegInfR;
+    int bi = n;
+    for (int e = lane; e < n; e += 64)
+      if (v[e] > b) {
+        b = v[e];
+        bi = e;
+      }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ob = __shfl_xor(b, o, 64);
+      const int oi = __shfl_xor(bi, o, 64);
+      if (ob > b || (ob == b && oi < bi)) {
+        b = ob;
+        bi = oi;
+      }
+    }
+    return bi;
+  };
+  if (groups > 0) {
+    const int per = E / groups;
+    for (int g = lane; g < groups; g += 64) {
+      float m = kNegInfR;
+      for (int e = g * per; e < (g + 1) * per; ++e) m = fmaxf(m, ch[e]);
+      gr[g] = m;
+    }
+    __syncthreads();
+    uint64_t kept[4] = {0, 0, 0, 0};                   // groups <= 256
+    for (int a = 0; a < keep; ++a) {
+      const int g = best_of(gr, groups);
+      if (g < groups) {
+#pragma unroll
+        for (int w = 0; w < 4; ++w)
+          if ((g >> 6) == w) kept[w] |= 1ull << (g & 63);
+        if (lane == 0) gr[g] = kNegInfR;
+      }
+      __syncthreads();
+    }
+    for (int e = lane; e < E; e += 64) {
+      const int g = e / per;
+      uint64_t w = kept[0];
+#pragma unroll
+      for (int k = 1; k < 4; ++k)
+        if ((g >> 6) == k) w = kept[k];
+      if (!((w >> (g & 63)) & 1)) ch[e] = kNegInfR;
+    }
+    __syncthreads();
+  }
+  float id_sum = 0.f;
+  for (int a = 0; a < top; ++a) {
+    const int e = best_of(ch, E);
+    const bool any = e < E;                            // non-finite logits: nothing to choose
+    const bool is_real = any && e < real;
+    const float w = any ? sc[e] * scale : 0.f;
+    if (any && !is_real) id_sum += w;
+    if (lane == 0) {
+      ids[(int64_t)t * top + a] = is_real ? e : real;
+      weights[(int64_t)t * top + a] = is_real ? w : 0.f;
+    }
+    __syncthreads();
+    if (lane == 0 && any) ch[e] = kNegInfR;
+    __syncthreads();
+  }
+  if (lane == 0 && ident != nullptr) ident[t] = id_sum;
 }
 
 // act[p, f] = silu(Wg[e] . x_t) * (Wu[e] . x_t) for pair p = t * top + k, e = ids[p].
@@ -133,6 +236,17 @@ void launch_moe_route_grouped(const float* z, const float* corr, int T, int E, i
   if (T == 0) return;
   hipLaunchKernelGGL(moe_route_grouped_kernel, dim3((T + 255) / 256), dim3(256), 0, s, z, corr, T,
                      E, top, groups, keep, ids, weights);
+}
+
+bool moe_route_softmax_ok(int E, int groups) { return E <= 4096 && groups <= 256; }
+
+void launch_moe_route_softmax(const float* z, int64_t zs, const float* corr, int T, int E, int real,
+                              int top, int groups, int keep, float scale, int32_t* ids,
+                              float* weights, float* ident, hipStream_t s) {
+  if (T == 0) return;
+  const size_t lds = (size_t)(2 * E + groups) * 4;
+  hipLaunchKernelGGL(moe_route_softmax_kernel, dim3(T), dim3(64), lds, s, z, zs, corr, E, real, top,
+                     groups, keep, scale, ids, weights, ident);
 }
 
 void launch_moe_pair_up(bool f32, const void* h, int64_t h_stride, const int32_t* ids,

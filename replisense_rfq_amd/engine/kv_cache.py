@@ -64,14 +64,15 @@ class LayeredKVCache:
       window_attention   K and V pools like ``attention``;
       rope_latent_attention   like ``latent_attention`` with rows ``[latent | rotated key
                          part]``, ``kv_rank + rot_dim`` wide;
-      wkv, gla, channel_delta   no pages.
+      wkv, gla, channel_delta, mlstm   no pages.
     Per-sequence state lives in slots; a sequence owns one while it runs (native core).  Every
     state pool is double buffered: a step reads half ``gen & 1`` of the slot and writes the
     other, so rows of one launch never read what the launch writes.  ``state``: the input
     convolutions' last inputs ``[L, 2 sublayers, 2 * slots, taps - 1, d]`` fp32;
     ``layer_state[i]``: name -> ``[2 * slots, ...]`` fp32 for what ``cfg.state_shapes(i)``
     lists (a wkv layer's matrices and its previous input row; a gla or channel_delta
-    layer's matrices, and the convolutions' last inputs; with ``cfg.token_shift`` every
+    layer's matrices, and the convolutions' last inputs; an mlstm layer's matrices, key sums
+    and running maxima; with ``cfg.token_shift`` every
     layer's previous normed input row)."""
 
     def __init__(self, cfg, num_blocks: int, device, num_slots: int, block_size: int = 32,

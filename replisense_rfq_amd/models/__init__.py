@@ -20,4 +20,8 @@ def layered_model_class(architecture: str):
         from .nutitar import NutitarLM
 
         return NutitarLM
+    if architecture == "Modepel":
+        from .modepel import ModepelLM
+
+        return ModepelLM
     raise KeyError(f"no model class for architecture {architecture!r}")

@@ -114,7 +114,12 @@ class MixerSpec:
     whole projection (``all``), half-split rotation of the first ``rot_dims`` dimensions,
     position i sees j <= i with i - j < ``window`` or j < ``keep_first`` (window 0: plain
     causal); ``weights`` = ``softmax`` or ``sigmoid`` (unnormalised, with a per-head bias);
-    ``bias``: the projections have biases; ``v_is_k``: the values are the keys as projected.
+    ``bias``: the projections have biases; ``v_is_k``: the values are the keys as projected;
+    ``sink`` = ``unit``: the softmax's denominator holds an added 1; ``v_mix``: the values are
+    blended with those of the first layer that has it (which stay as projected); ``out_gate``: a
+    sigmoid gate per output.
+    ``mlstm``: ``heads`` recurrent heads with a ``dim`` x ``vdim`` matrix memory, a ``dim``-wide
+    key sum and a running maximum, exponential gates whose logits are capped at ``gate_cap``.
     The rotating kinds take their frequencies from ``rot_base`` and ``rot_scaling``: () for
     none, ("yarn", factor, original, fast, slow) or ("banded", factor, original, low,
     high)."""
@@ -141,6 +146,10 @@ class MixerSpec:
     weights: str = "softmax"
     bias: bool = False
     v_is_k: bool = False
+    sink: str = ""
+    v_mix: bool = False
+    out_gate: bool = False
+    gate_cap: float = 0.0
 
     @property
     def group(self) -> int:
@@ -155,7 +164,11 @@ class MlpSpec:
     ``shared_ff`` (0: none); ``router`` = ``softmax_top``: the ``top`` largest router logits
     (with a bias), weighted by the softmax over the chosen logits only.  ``gelu``: up
     projection, exact gelu, down projection.  ``xielu``: up projection, a quadratic / exponential
-    unit with two learned numbers, down projection."""
+    unit with two learned numbers, down projection.  ``polynorm``: up projection, a weighted sum of
+    normed powers, down projection.  ``router`` = ``grouped_softmax``: softmax over the experts and
+    ``identity`` further router outputs whose "expert" is the input itself, a correction in the
+    choice, groups ranked by their largest choice score, weights times ``router_scale``; the shared
+    expert is then gated by one logit per token."""
     kind: str = "dense"
     ff: int = 256
     limit: float = 7.0
@@ -165,6 +178,8 @@ class MlpSpec:
     keep: int = 0
     shared_ff: int = 0
     router: str = "grouped_sigmoid"
+    identity: int = 0
+    router_scale: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -246,7 +261,9 @@ class LayeredConfig:
                 n += d * (m.kv_rank + m.rot_dim) if m.kv_from < 0 else 0
             elif m.kind == "window_attention":
                 n += d * (m.heads * m.dim + m.kv_heads * (m.dim + (0 if m.v_is_k else m.vdim)))
-                n += m.heads * m.vdim * d
+                n += m.heads * m.vdim * d * (2 if m.out_gate else 1)
+            elif m.kind == "mlstm":
+                n += d * m.heads * (2 * m.dim + 3 * m.vdim + 2)
             elif m.kind == "gla":
                 n += 2 * d * m.heads * (m.dim + m.vdim) + m.heads * m.vdim * d
                 n += self.decay_rank * (d + m.heads * m.dim)
@@ -257,9 +274,9 @@ class LayeredConfig:
                 n += 5 * d * m.heads * m.dim + 2 * d * self.decay_rank
             f = ly.mlp
             if f is not None and f.kind == "moe":
-                n += 3 * d * (f.ff * f.experts + f.shared_ff) + d * f.experts
+                n += 3 * d * (f.ff * f.experts + f.shared_ff) + d * (f.experts + f.identity)
             elif f is not None:
-                n += (2 if f.kind in ("gelu", "xielu") else 3) * d * f.ff
+                n += (2 if f.kind in ("gelu", "xielu", "polynorm") else 3) * d * f.ff
         return n + 2 * self.vocab_size * d + d
 
     def kv_bytes_per_token(self, tp: int = 1, dtype_bytes: int = 2) -> int:
@@ -286,6 +303,8 @@ class LayeredConfig:
             return {"prev": (self.hidden,)}
         if m.kind == "wkv":
             return {"wkv": (m.heads, m.dim, m.dim), "prev": (self.hidden,)}
+        if m.kind == "mlstm":
+            return {"S": (m.heads, m.dim, m.vdim), "n": (m.heads, m.dim), "m": (m.heads,)}
         if m.kind == "gla":
             return {"S": (m.heads, m.dim, m.vdim)}
         if m.kind == "channel_delta":
@@ -489,6 +508,82 @@ def nutitar_from_json(d: dict, name: str | None = None) -> LayeredConfig:
                          residual_mult=float(d["residual_mult"]), token_shift=True)
 
 
+def modepel_from_json(d: dict, name: str | None = None) -> LayeredConfig:
+    """config.json of a Modepel checkpoint: vocab, width, norm.eps and ``layers``: type
+    ``attention`` (heads, kv_heads, dim, vdim, scale, rot.dims, rot.base, v_mix) or ``mlstm``
+    (heads, dim, vdim, gate_cap), each with an ``mlp`` of kind ``dense`` (ff), ``moe`` (expert.ff,
+    router.experts / identity / top / scale / groups.count / groups.keep, shared.ff) or null."""
+    layers, blended = [], None
+    for i, ly in enumerate(d["layers"]):
+        m, kind = ly["mixer"], ly["type"]
+        if kind == "attention":
+            rot = m.get("rot") or {}
+            mixer = MixerSpec("window_attention", int(m["heads"]), int(m["kv_heads"]), int(m["dim"]),
+                              int(m["vdim"]), float(m["scale"]), rot_dims=int(rot.get("dims", 0)),
+                              rot_base=float(rot.get("base", 10000.0)), bias=True, sink="unit",
+                              v_mix=bool(m.get("v_mix", False)), out_gate=True)
+            if mixer.heads % mixer.kv_heads:
+                raise ValueError(f"layer {i}: heads must be a multiple of kv_heads")
+            if mixer.rot_dims % 2 or mixer.rot_dims > mixer.dim:
+                raise ValueError(f"layer {i}: rot.dims must be even and at most dim")
+            if mixer.v_mix:
+                blended = blended or (i, mixer.kv_heads, mixer.vdim)
+                if (mixer.kv_heads, mixer.vdim) != blended[1:]:
+                    raise ValueError(f"layer {i}: its values cannot be blended with layer {blended[0]}'s: "
+                                     f"other heads or sizes")
+        elif kind == "mlstm":
+            mixer = MixerSpec("mlstm", int(m["heads"]), int(m["heads"]), int(m["dim"]), int(m["vdim"]),
+                              float(m["dim"]) ** -0.5, gate_cap=float(m["gate_cap"]))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+        f = ly.get("mlp")
+        mlp = None
+        if f is not None and f.get("kind") == "dense":
+            mlp = MlpSpec("polynorm", int(f["ff"]), 0.0)
+        elif f is not None and f.get("kind") == "moe":
+            r = f["router"]
+            g = r.get("groups") or {}
+            E, I, top = int(r["experts"]), int(r.get("identity") or 0), int(r["top"])
+            count, keep = int(g.get("count", 0)), int(g.get("keep", 0))
+            if count and ((E + I) % count or not 0 < keep <= count):
+                raise ValueError(f"layer {i}: {E + I} router outputs do not form {count} equal groups")
+            if not 0 < top <= (keep * ((E + I) // count) if count else E + I):
+                raise ValueError(f"layer {i}: the kept groups hold fewer than top experts")
+            mlp = MlpSpec("moe", int(f["expert"]["ff"]), 0.0, E, top, count, keep,
+                          int((f.get("shared") or {}).get("ff", 0)), "grouped_softmax", I,
+                          float(r.get("scale", 1.0)))
+        elif f is not None:
+            raise ValueError(f"layer {i}: unknown feed-forward kind {f.get('kind')!r}")
+        layers.append(LayerSpec(mixer, mlp))
+    return LayeredConfig(name=name or d["architecture"].lower(), architecture=d["architecture"],
+                         vocab_size=int(d["vocab"]), hidden=int(d["width"]), layers=tuple(layers),
+                         rms_eps=float(d["norm"]["eps"]), canon_taps=0,
+                         max_position=int(d.get("max_position", 8192)))
+
+
+def modepel_layers(order, heads, kv_heads, dim, vdim, ff, experts=0, top=0, expert_ff=0, identity=0,
+                   groups=0, keep=0, shared_ff=0, router_scale=1.0, rot_dims=None, rot_base=10000.0,
+                   scale=None, gate_cap=15.0, rec_heads=None, rec_dim=None, rec_vdim=None, moe_from=1):
+    """Layers of the kinds named in ``order`` ("a" attention, "m" mlstm); with experts the layers
+    from ``moe_from`` on have a mixture, the others (with ff > 0) the polynomial unit."""
+    rh, rd, rv = rec_heads or heads, rec_dim or dim, rec_vdim or vdim
+    out = []
+    for i, c in enumerate(order):
+        if c == "a":
+            m = MixerSpec("window_attention", heads, kv_heads, dim, vdim, scale or dim ** -0.5,
+                          rot_dims=dim if rot_dims is None else rot_dims, rot_base=rot_base, bias=True,
+                          sink="unit", v_mix=True, out_gate=True)
+        else:
+            m = MixerSpec("mlstm", rh, rh, rd, rv, rd ** -0.5, gate_cap=gate_cap)
+        if experts and i >= moe_from:
+            f = MlpSpec("moe", expert_ff, 0.0, experts, top, groups, keep, shared_ff, "grouped_softmax",
+                        identity, router_scale)
+        else:
+            f = MlpSpec("polynorm", ff, 0.0) if ff else None
+        out.append(LayerSpec(m, f))
+    return tuple(out)
+
+
 def nutitar_layers(order, heads, kv_heads, dim, vdim, ff, kv_rank=0, rot_dim=0, window=0,
                    keep_first=0, rot_dims=None, rot_base=10000.0, yarn=(), banded=(), scale=None,
                    latent_heads=None, latent_dim=None):
@@ -590,12 +685,21 @@ TINY_NUTITAR = LayeredConfig("tiny-nutitar", architecture="Nutitar", vocab_size=
                                                    rot_base=5000.0, yarn=(3.0, 64.0, 16.0, 2.0),
                                                    banded=(3.0, 48.0, 1.0, 3.0), latent_heads=5,
                                                    latent_dim=20))
+# both mixers and all three feed-forwards; sizes that differ wherever the design allows
+TINY_MODEPEL = LayeredConfig("tiny-modepel", architecture="Modepel", vocab_size=304, hidden=96,
+                             canon_taps=0, rms_eps=1e-6,
+                             layers=modepel_layers("amam", 6, 2, 16, 24, 160, experts=5, top=3,
+                                                   expert_ff=40, identity=3, groups=4, keep=3,
+                                                   shared_ff=56, router_scale=1.3, rot_dims=8,
+                                                   rot_base=5000.0, gate_cap=9.0, rec_heads=3,
+                                                   rec_dim=20, rec_vdim=28))
 CONFIGS.update({c.name: c for c in (TINY_LIVISUN, LIVISUN_8B, TINY_NUMALORN, TINY_BILOLIX,
-                                    TINY_NUTITAR)})
+                                    TINY_NUTITAR, TINY_MODEPEL)})
 
 # config.json "architecture" -> reader
 ARCHITECTURES = {"Livisun": LayeredConfig.from_json, "Numalorn": numalorn_from_json,
-                 "Bilolix": bilolix_from_json, "Nutitar": nutitar_from_json}
+                 "Bilolix": bilolix_from_json, "Nutitar": nutitar_from_json,
+                 "Modepel": modepel_from_json}
 
 
 def load_config(path: str):

@@ -80,12 +80,14 @@ class MoEBuffers:
 
 def moe_mlp(x: torch.Tensor, router_w: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor,
             topk: int, bufs: MoEBuffers | None, out: torch.Tensor | None = None,
-            expert_offset: int = 0, routing=None) -> torch.Tensor:
+            expert_offset: int = 0, routing=None, spare: bool = False) -> torch.Tensor:
     """x [T, d] -> [T, d].  w13 [E, 2F, d] (gate|up), w2 [E, d, F], router_w [E_all, d].
 
     ``routing``: a callable (weights [T, topk] fp32, ids [T, topk] int32) that fills both for
     this step's rows in place of the softmax top-k router (models with a router of their own;
-    GPU only); the alignment, expert GEMMs and weighted combine are the same.
+    GPU only); the alignment, expert GEMMs and weighted combine are the same.  ``spare``: the
+    router leaves pairs that no expert computes (identity experts) as id E with weight 0; they
+    go to a segment of their own that no kernel touches, and ``bufs`` is sized for E + 1.
 
     Expert parallelism: when this rank holds experts [expert_offset, expert_offset +
     E) of E_all, pairs routed elsewhere are sent to a dummy expert segment that no
@@ -95,15 +97,15 @@ def moe_mlp(x: torch.Tensor, router_w: torch.Tensor, w13: torch.Tensor, w2: torc
     if not x.is_cuda:
         return ref.moe_forward(x, w13, w2, x @ router_w.t(), topk, expert_offset)
     E = w13.shape[0]
-    ep = E != router_w.shape[0]
+    ep = not spare and E != router_w.shape[0]
     assert bufs is not None and T <= bufs.max_tokens
     out = torch.empty_like(x) if out is None else out
     # buffers are sliced to this step's token count but keep their capacity-based
     # padding so the grouped GEMM grid is fixed for a given bucket
     n = T * topk
     w, ids = bufs.weights[:T], bufs.ids[:T]
-    if ep:
-        E = E + 1                  # + the dummy segment for remote experts
+    if ep or spare:
+        E = E + 1                  # + the dummy segment for remote experts / identity pairs
     if T <= SKINNY_MAX_TOKENS:
         # decode / short-extend steps: router GEMV + top-k in one kernel, stream only
         # the routed experts' weights, gather rows on the fly, SwiGLU fused into w13

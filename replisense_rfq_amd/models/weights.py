@@ -299,6 +299,8 @@ def load_layered_safetensors(path: str, cfg, device, dtype=torch.bfloat16) -> di
         return _bilolix_assemble(ck.full, lambda k: k in ck, cfg, device, dtype)
     if cfg.architecture == "Nutitar":
         return _nutitar_assemble(ck.full, lambda k: k in ck, cfg, device, dtype)
+    if cfg.architecture == "Modepel":
+        return _modepel_assemble(ck.full, lambda k: k in ck, cfg, device, dtype)
     w = {"embed": ck.full("embed").to(dtype).to(device), "lm_head": ck.full("head").to(dtype).to(device),
          "final_norm": ck.full("final.norm").float().to(device), "vocab_start": 0, "layers": []}
     for i, ly in enumerate(cfg.layers):
@@ -860,5 +862,157 @@ def init_nutitar_weights(cfg, device, dtype=torch.bfloat16, seed: int = 0,
 
 def nutitar_from_full(full: dict, cfg, device, dtype=torch.bfloat16) -> dict:
     w = _nutitar_assemble(lambda k: full[k], lambda k: k in full, cfg, device, dtype)
+    w["full"] = full
+    return w
+
+
+# --------------------------------------------------------------------------
+# Modepel.  Checkpoint names:
+#   embed, head [V, d]; final.norm, l<i>.norm1 | norm1b (| norm2 | norm2b) [] (one number each)
+#   attention: l<i>.mix.q [H*dim, d]  .k [G*dim, d]  .v [G*vdim, d] (+ .b)  .g [H*vdim, d]
+#     .vmix [] (layers that blend values)  .o [d, H*vdim]
+#   mlstm: l<i>.mix.q | k [H*dim, d]  .v | g [H*vdim, d]  .i | f [H, d] (+ .b)  .norm [H*vdim]
+#     .o [d, H*vdim]
+#   dense: l<i>.mlp.up [F, d]  .down [d, F]  .act [4]
+#   moe: l<i>.mlp.router [E + I, d]  .correction [E + I]  .e<j>.gate | up [F, d]  .e<j>.down [d, F]
+#     .shared.gate | up | down  .shared.sg [1, d]
+# Loaded layout per layer: one fused input projection "proj" (q | k | v | gate rows; the first
+# three segments' bias "proj_b" in fp32), the recurrence's two gate projections in one matrix
+# "zif" with its bias, router and shared-gate rows in one matrix "router" (their products leave in
+# fp32), gains and coefficients as Python floats.
+def _modepel_assemble(get, has, cfg, device, dtype) -> dict:
+    d = cfg.hidden
+
+    def mat(name, rows, cols):
+        t = get(name)
+        if tuple(t.shape) != (rows, cols):
+            raise ValueError(f"tensor {name}: shape {tuple(t.shape)}, expected {(rows, cols)}")
+        return t.to(dtype)
+
+    def vec(name, *shape):
+        t = get(name)
+        if tuple(t.shape) != tuple(shape):
+            raise ValueError(f"tensor {name}: shape {tuple(t.shape)}, expected {tuple(shape)}")
+        return t.float().contiguous().to(device)
+
+    def num(name):
+        t = get(name)
+        if t.numel() != 1:
+            raise ValueError(f"tensor {name}: shape {tuple(t.shape)}, expected one number")
+        return float(t.float())
+
+    V = cfg.vocab_size
+    w = {"embed": mat("embed", V, d).to(device), "lm_head": mat("head", V, d).to(device),
+         "final_norm": num("final.norm"), "vocab_start": 0, "layers": []}
+    for i, ly in enumerate(cfg.layers):
+        p, m, lw = f"l{i}.mix.", ly.mixer, LayerWeights()
+        lw["norm1"], lw["norm1b"] = num(f"l{i}.norm1"), num(f"l{i}.norm1b")
+        H, G, dim, vd = m.heads, m.kv_heads, m.dim, m.vdim
+        if m.kind not in ("window_attention", "mlstm"):
+            raise ValueError(f"layer {i}: no weights known for mixer {m.kind!r}")
+        rows = {"q": H * dim, "k": G * dim, "v": G * vd, "g": H * vd}
+        lw["proj"] = torch.cat([mat(p + n, rows[n], d) for n in "qkvg"], 0).contiguous().to(device)
+        if m.kind == "window_attention":
+            lw["proj_b"] = torch.cat([vec(p + n + ".b", rows[n]) for n in "qkv"]).contiguous()
+            lw["vmix"] = num(p + "vmix") if m.v_mix else 0.0
+            lw["sink"] = torch.zeros(H, dtype=torch.float32, device=device)   # exp(0) = the added 1
+        else:
+            lw["zif"] = torch.cat([mat(p + "i", H, d), mat(p + "f", H, d)], 0).contiguous().to(device)
+            lw["zif_b"] = torch.cat([vec(p + "i.b", H), vec(p + "f.b", H)]).contiguous()
+            lw["gn"] = vec(p + "norm", H * vd)
+        lw["o"] = mat(p + "o", d, H * vd).contiguous().to(device)
+        f, q = ly.mlp, f"l{i}.mlp."
+        if f is not None:
+            lw["norm2"], lw["norm2b"] = num(f"l{i}.norm2"), num(f"l{i}.norm2b")
+        if f is not None and f.kind == "moe":
+            n = f.experts + f.identity
+            parts = [mat(q + "router", n, d)]
+            if f.shared_ff:
+                parts.append(mat(q + "shared.sg", 1, d))
+                lw["shared_gu"] = torch.cat([mat(q + "shared.gate", f.shared_ff, d),
+                                             mat(q + "shared.up", f.shared_ff, d)], 0).contiguous().to(device)
+                lw["shared_down"] = mat(q + "shared.down", d, f.shared_ff).contiguous().to(device)
+            lw["router"] = torch.cat(parts, 0).contiguous().to(device)
+            lw["correction"] = vec(q + "correction", n)
+            lw["w13"] = torch.stack([torch.cat([mat(f"{q}e{e}.gate", f.ff, d), mat(f"{q}e{e}.up", f.ff, d)], 0)
+                                     for e in range(f.experts)]).contiguous().to(device)
+            lw["w2e"] = torch.stack([mat(f"{q}e{e}.down", d, f.ff) for e in range(f.experts)]) \
+                .contiguous().to(device)
+        elif f is not None:
+            lw["up"] = mat(q + "up", f.ff, d).contiguous().to(device)
+            lw["down"] = mat(q + "down", d, f.ff).contiguous().to(device)
+            lw["poly"] = tuple(float(x) for x in vec(q + "act", 4).cpu())
+        w["layers"].append(lw)
+    return w
+
+
+def init_modepel_weights(cfg, device, dtype=torch.bfloat16, seed: int = 0,
+                         keep_full: bool = True) -> dict:
+    """Seeded random Modepel weights under the checkpoint's names (tests and benchmarks):
+    projections scaled so that activations stay O(1); gains, biases, blends, gate biases (slow and
+    fast forgetting side by side), corrections and the unit's numbers away from their neutral
+    values so that each shows in the logits.  ``keep_full`` False (benchmark sizes): drawn on the
+    device, the name -> tensor dict is not kept."""
+    d, full = cfg.hidden, {}
+
+    def rnd(name, shape, std, mean=0.0):
+        if keep_full:
+            t = _randn(shape, std, (seed, name), "cpu", torch.float32) + mean
+            full[name] = t.to(torch.bfloat16).float()
+        else:
+            full[name] = (_randn(shape, std, (seed, name), device, torch.float32) + mean).to(torch.bfloat16)
+        return full[name]
+
+    rnd("embed", (cfg.vocab_size, d), 1.0)
+    rnd("head", (cfg.vocab_size, d), 2.0 * d ** -0.5)
+    rnd("final.norm", (), 0.2, 1.0)
+    for i, ly in enumerate(cfg.layers):
+        p, m = f"l{i}.mix.", ly.mixer
+        H, G, dim, vd = m.heads, m.kv_heads, m.dim, m.vdim
+        rnd(f"l{i}.norm1", (), 0.2, 1.1)
+        rnd(f"l{i}.norm1b", (), 0.2, 0.9)
+        rnd(p + "q", (H * dim, d), 2.0 * d ** -0.5)
+        rnd(p + "k", (G * dim, d), 2.0 * d ** -0.5)
+        rnd(p + "v", (G * vd, d), 1.5 * d ** -0.5)
+        rnd(p + "g", (H * vd, d), 2.0 * d ** -0.5)
+        if m.kind == "mlstm":
+            rnd(p + "i", (H, d), d ** -0.5)
+            rnd(p + "f", (H, d), d ** -0.5)
+            rnd(p + "i.b", (H,), 1.5)
+            rnd(p + "f.b", (H,), 2.0, 3.0)
+            rnd(p + "norm", (H * vd,), 0.2, 1.0)
+        else:
+            for n, c in (("q", H * dim), ("k", G * dim), ("v", G * vd)):
+                rnd(p + n + ".b", (c,), 0.3)
+            if m.v_mix:
+                rnd(p + "vmix", (), 0.15, 0.4)
+        rnd(p + "o", (d, H * vd), (H * vd) ** -0.5)
+        f, q = ly.mlp, f"l{i}.mlp."
+        if f is not None:
+            rnd(f"l{i}.norm2", (), 0.2, 1.1)
+            rnd(f"l{i}.norm2b", (), 0.2, 0.9)
+        if f is not None and f.kind == "moe":
+            rnd(q + "router", (f.experts + f.identity, d), 2.0 * d ** -0.5)
+            rnd(q + "correction", (f.experts + f.identity,), 0.2, -0.5)
+            for e in range(f.experts):
+                rnd(f"{q}e{e}.gate", (f.ff, d), d ** -0.5)
+                rnd(f"{q}e{e}.up", (f.ff, d), d ** -0.5)
+                rnd(f"{q}e{e}.down", (d, f.ff), f.ff ** -0.5)
+            if f.shared_ff:
+                rnd(q + "shared.gate", (f.shared_ff, d), d ** -0.5)
+                rnd(q + "shared.up", (f.shared_ff, d), d ** -0.5)
+                rnd(q + "shared.down", (d, f.shared_ff), f.shared_ff ** -0.5)
+                rnd(q + "shared.sg", (1, d), 1.5 * d ** -0.5)
+        elif f is not None:
+            rnd(q + "up", (f.ff, d), d ** -0.5)
+            rnd(q + "down", (d, f.ff), f.ff ** -0.5)
+            rnd(q + "act", (4,), 0.3, 0.5)
+    if not keep_full:
+        return _modepel_assemble(lambda k: full.pop(k), lambda k: k in full, cfg, device, dtype)
+    return modepel_from_full(full, cfg, device, dtype)
+
+
+def modepel_from_full(full: dict, cfg, device, dtype=torch.bfloat16) -> dict:
+    w = _modepel_assemble(lambda k: full[k], lambda k: k in full, cfg, device, dtype)
     w["full"] = full
     return w

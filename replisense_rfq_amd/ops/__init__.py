@@ -1409,16 +1409,16 @@ def rotary_scaled_freq(rot_dims: int, base: float, scaling: tuple = (), device="
 def qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all: bool, k_norm_n: int, eps: float,
                           positions, inv_freq, rot_mult: float, q_rot_off: int, k_rot_off: int,
                           slot_mapping, k_cache, v_cache, H: int, G: int, qw: int, kw: int, vdim: int,
-                          v_mode: int, q_out):
+                          v_mode: int, q_out, v_in=None, v_take: float = 0.0, v_out=None):
     if _gpu(proj):
         _native.mix_ops().qk_norm_rotary_append(
             proj, bias, q_norm_w, k_norm_w, bool(norm_all), int(k_norm_n), float(eps), positions,
             inv_freq, float(rot_mult), int(q_rot_off), int(k_rot_off), slot_mapping, k_cache,
-            v_cache, H, G, qw, kw, vdim, int(v_mode), q_out)
+            v_cache, H, G, qw, kw, vdim, int(v_mode), q_out, v_in, float(v_take), v_out)
     else:
         ref.qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all, k_norm_n, eps, positions,
                                   inv_freq, rot_mult, q_rot_off, k_rot_off, slot_mapping, k_cache,
-                                  v_cache, H, G, qw, kw, vdim, v_mode, q_out)
+                                  v_cache, H, G, qw, kw, vdim, v_mode, q_out, v_in, v_take, v_out)
     return q_out
 
 
@@ -1440,7 +1440,8 @@ def attn_keep_window(q, k_cache, v_cache, vdim: int, block_tables, q_start, q_le
     ``short_rows`` > 0: every sequence has at most that many rows (a decode section); the
     kernel then runs one workgroup per (sequence, key/value head) over one pass through the
     pages where the sizes fit its LDS.  Otherwise bf16 pages whose sizes the MFMA tiles cover
-    run on them unless ``mfma`` is False (the FMA work-item kernel)."""
+    run on them unless ``mfma`` is False (the FMA work-item kernel).  ``gate``: logits [T, H]
+    (one per head) or [T, H vdim] (one per output)."""
     if _gpu(q):
         _native.mix_ops().attn_keep_window(q, k_cache, v_cache, int(vdim), block_tables, q_start,
                                            q_len, kv_len, work_seq, work_qblk, head_bias, gate, out,
@@ -1459,4 +1460,71 @@ def xielu_rows(x, alpha_p: float, alpha_n: float, out=None):
         _native.mix_ops().xielu_rows(x, float(alpha_p), float(alpha_n), out)
     else:
         ref.xielu_rows(x, alpha_p, alpha_n, out)
+    return out
+
+
+# ---------------------------------------------------------------------------
+# Norms with single gains around every sublayer, the polynomial norm unit, softmax routing with
+# identity experts, the matrix-memory recurrence (csrc/kernels/mix_gain.hip, mix_route.hip,
+# mix_mlstm.hip, mix_mlstm_mfma.hip; same library).
+def gain_sandwich(x, y=None, g_post: float = 1.0, g_pre: float = 1.0, eps: float = 1e-6, out=None,
+                  y2=None, y2_logit=None, h_in=None, h_weight=None):
+    """Y = y + sigmoid(y2_logit) y2 + h_weight h_in (each term optional, either dtype; one logit
+    and one weight per row, fp32); x (fp32, in place) += g_post Y / rms(Y); ``out`` (either
+    dtype, optional) receives g_pre x / rms(x)."""
+    if _gpu(x):
+        _native.mix_ops().gain_sandwich(x, y, y2, y2_logit, h_in, h_weight, float(g_post),
+                                        float(g_pre), float(eps), out)
+    else:
+        ref.gain_sandwich(x, y, g_post, g_pre, eps, out, y2, y2_logit, h_in, h_weight)
+    return out
+
+
+def poly_norm_rows(x, coef, eps: float, out=None):
+    """a N(z) + b N(z^2) + c N(z^3) + e per row, coef = (a, b, c, e); may run in place."""
+    out = torch.empty_like(x) if out is None else out
+    if _gpu(x):
+        a, b, c, e = coef
+        _native.mix_ops().poly_norm_rows(x, float(a), float(b), float(c), float(e), float(eps), out)
+    else:
+        ref.poly_norm_rows(x, coef, eps, out)
+    return out
+
+
+def moe_route_softmax(z, correction, real: int, top: int, groups: int, keep: int, scale: float, ids,
+                      weights, ident=None):
+    """The first correction.numel() columns of z are the router's logits, the columns from
+    ``real`` on identity experts: a chosen one is left as id ``real`` with weight 0 and its weight
+    added to ident[t]."""
+    if _gpu(z):
+        _native.mix_ops().moe_route_softmax(z, correction, int(real), int(top), int(groups), int(keep),
+                                            float(scale), ids, weights, ident)
+    else:
+        ref.moe_route_softmax(z, correction, real, top, groups, keep, scale, ids, weights, ident)
+
+
+MLSTM_SCAN_ROWS = 128      # steps with more rows leave norm and gate to a row-parallel kernel
+MLSTM_CHUNK = os.environ.get("RFQ_MLSTM_CHUNK", "1") != "0"     # and run bf16 in chunks on MFMA tiles
+
+
+def mlstm_recurrence(q, k, v, z, zbias, cap: float, q_scale: float, gate, norm_w, eps: float, S, n, m,
+                     row_state, row_back, row_fwd, positions, out, run_rows=None,
+                     chunked: bool | None = None):
+    """q, k [T, H dim], v, gate [T, H vdim] (column slices of a projection), z [T, 2 H] fp32 raw
+    logits of the input gates and then the forget gates.  ``run_rows`` as for
+    gated_linear_recurrence.  On the GPU a bf16 step of more than MLSTM_SCAN_ROWS rows runs in
+    chunks of 64 tokens on MFMA tiles where the sizes fit, every other step token by token."""
+    if _gpu(out):
+        o = _native.mix_ops()
+        H, dim, vdim = S.shape[1:]
+        long = out.shape[0] > MLSTM_SCAN_ROWS if chunked is None else chunked
+        raw = None
+        if long or not o.mlstm_fused_ok(dim, vdim):
+            raw = torch.empty(out.shape, dtype=torch.float32, device=out.device)
+        o.mlstm_recurrence(q, k, v, z, zbias, float(cap), float(q_scale), gate, norm_w, float(eps), S, n, m,
+                           row_state, row_back, row_fwd, positions, run_rows, out, raw,
+                           bool(long and (MLSTM_CHUNK or chunked)))
+    else:
+        ref.mlstm_recurrence(q, k, v, z, zbias, cap, q_scale, gate, norm_w, eps, S, n, m, row_state,
+                             row_back, row_fwd, positions, out)
     return out

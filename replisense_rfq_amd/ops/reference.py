@@ -764,7 +764,7 @@ def _rotate_halves(x, positions, inv_freq, mult: float, off: int):
 def qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all: bool, k_norm_n: int, eps: float,
                           positions, inv_freq, rot_mult: float, q_rot_off: int, k_rot_off: int,
                           slot_mapping, k_cache, v_cache, H: int, G: int, qw: int, kw: int, vdim: int,
-                          v_mode: int, q_out) -> None:
+                          v_mode: int, q_out, v_in=None, v_take: float = 0.0, v_out=None) -> None:
     """Rows of proj are q [H, qw] | k [G, kw] (| v [G, vdim] with v_mode 0); ``bias`` (fp32, the
     row's width) is added first.  RMS norms with plain weights: over the whole q and the whole k
     projection (``norm_all``; weights [H qw], [G kw]) or per head, q over its qw entries
@@ -772,13 +772,14 @@ def qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all: bool, k_norm
     None means no norm.  Then the half-split rotation of entries rot_off .. rot_off + 2 n of
     every head.  q goes to q_out [T, H, qw] fp32; k rows into k_cache [blocks, G, BS, kw];
     values into v_cache [blocks, G, BS, vdim]: v_mode 0 the v columns, 1 the keys as projected
-    (before norm and rotation), 2 none."""
+    (before norm and rotation), 2 none.  ``v_out`` [T, G vdim] fp32 receives the values as
+    projected; with ``v_in`` [T, G vdim] fp32 the cached ones are (1 - v_take) v + v_take v_in."""
     T = proj.shape[0]
     if T == 0:
         return
     x = proj.float()
     if bias is not None:
-        x = x + bias.float()
+        x = x[:, :bias.numel()] + bias.float()
     nq, nk = H * qw, G * kw
     q, k = x[:, :nq], x[:, nq:nq + nk]
     raw_k = k.reshape(T, G, kw)
@@ -800,6 +801,10 @@ def qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all: bool, k_norm
     if k_cache is None or G == 0:
         return
     v = x[:, nq + nk:nq + nk + G * vdim].reshape(T, G, vdim) if v_mode == 0 else raw_k
+    if v_out is not None:
+        v_out.copy_(v.reshape(T, G * vdim))
+    if v_in is not None:
+        v = (1.0 - v_take) * v + v_take * v_in.view(T, G, vdim)
     BS = k_cache.shape[2]
     for t in range(T):
         s = int(slot_mapping[t])
@@ -816,7 +821,8 @@ def attn_keep_window(q, k_cache, v_cache, vdim: int, block_tables, q_start, q_le
     i - j < window or j < keep_first (window 0: every j <= i).  Weights: softmax over the
     visible keys, with exp(head_bias[h]) added to the denominator when head_bias is given; or
     (``sigmoid``) sigmoid(score + head_bias[h]) per visible key, not normalised.  ``gate``
-    [T, H]: the head's output is multiplied by sigmoid(gate).  out [T, H vdim]."""
+    [T, H] (one logit per head) or [T, H vdim] (one per output): the output is multiplied by
+    sigmoid(gate).  out [T, H vdim]."""
     H = q.shape[1]
     G = k_cache.shape[1]
     rep = H // G
@@ -841,7 +847,7 @@ def attn_keep_window(q, k_cache, v_cache, vdim: int, block_tables, q_start, q_le
             p = torch.softmax(s, -1)[..., :kl]
         o = torch.einsum("hqk,hkd->qhd", p, v)
         if gate is not None:
-            o = o * torch.sigmoid(gate[t0:t0 + ql].float())[:, :, None]
+            o = o * torch.sigmoid(gate[t0:t0 + ql].float()).reshape(ql, H, -1)
         out[t0:t0 + ql].copy_(o.reshape(ql, -1).to(out.dtype))
 
 
@@ -851,3 +857,98 @@ def xielu_rows(x, alpha_p: float, alpha_n: float, out) -> None:
     zn = torch.clamp(z, max=0.0)
     out.copy_(torch.where(z > 0, alpha_p * z * z + 0.5 * z,
                           alpha_n * (torch.expm1(zn) - zn) + 0.5 * zn).to(out.dtype))
+
+
+# ---------------------------------------------------------------------------
+# Norms with single gains around every sublayer, the polynomial norm unit, softmax routing with
+# identity experts, the matrix-memory recurrence.
+def gain_sandwich(x, y, g_post: float, g_pre: float, eps: float, out, y2=None, y2_logit=None, h_in=None,
+                  h_weight=None) -> None:
+    """x (fp32, in place) += g_post * rms(y + sigmoid(y2_logit) y2 + h_weight h_in); with ``out``:
+    out = g_pre * rms(x) in out's dtype (which may be h_in)."""
+    parts = []
+    if y is not None:
+        parts.append(y.float())
+    if y2 is not None:
+        parts.append(torch.sigmoid(y2_logit.float())[:, None] * y2.float())
+    if h_in is not None:
+        parts.append(h_weight.float()[:, None] * h_in.float())
+    if parts:
+        x += _rms(sum(parts), eps) * g_post
+    if out is not None:
+        out.copy_((_rms(x, eps) * g_pre).to(out.dtype))
+
+
+def poly_norm_rows(x, coef, eps: float, out) -> None:
+    a, b, c, e = (float(v) for v in coef)
+    z = x.float()
+    out.copy_((a * _rms(z, eps) + b * _rms(z * z, eps) + c * _rms(z * z * z, eps) + e).to(out.dtype))
+
+
+def moe_route_softmax(z, correction, real: int, top: int, groups: int, keep: int, scale: float, ids,
+                      weights, ident) -> None:
+    """s = softmax(z) over all columns; chosen by s + correction inside the ``keep`` groups (of
+    ``groups`` equal groups of neighbours; 0 = no limit) with the largest choice score; weights =
+    scale * s of the chosen.  Columns from ``real`` on are identity experts: id ``real``, weight 0,
+    their weights summed in ident.  Ties go to the lower index."""
+    T, n = z.shape[0], correction.numel()
+    s = torch.softmax(z[:, :n].float(), -1)
+    choice = s + correction.float()
+    if groups > 0:
+        per = n // groups
+        grp = choice.view(T, groups, per)
+        kept = torch.zeros(T, groups, dtype=torch.bool)
+        order = torch.sort(grp.max(-1).values, dim=-1, descending=True, stable=True).indices[:, :keep]
+        kept.scatter_(1, order, True)
+        choice = torch.where(kept[:, :, None].expand(T, groups, per), grp,
+                             torch.full_like(grp, float("-inf"))).reshape(T, n)
+    idx = torch.sort(choice, dim=-1, descending=True, stable=True).indices[:, :top]
+    wt = s.gather(1, idx) * scale
+    same = idx >= real
+    ids.copy_(torch.where(same, torch.full_like(idx, real), idx).to(ids.dtype))
+    weights.copy_(torch.where(same, torch.zeros_like(wt), wt))
+    if ident is not None:
+        ident.copy_((wt * same).sum(-1))
+
+
+def mlstm_recurrence(q, k, v, z, zbias, cap: float, q_scale: float, gate, norm_w, eps: float, S, n, m,
+                     row_state, row_back, row_fwd, positions, out) -> None:
+    """Per head a dim x vdim state S, a key sum n and a running maximum m (fp32, zero at the
+    start), token by token inside each scheduled run:
+        li = cap tanh((zi + bi) / cap) ;  lf = log sigmoid(cap tanh((zf + bf) / cap))
+        m' = max(lf + m, li) ;  S <- e^(lf + m - m') S + e^(li - m') k v^T ;  n likewise with k
+        o = q_scale S^T q / (max(|q_scale n . q|, e^-m') + 1e-6)
+    out = o / rms(o) * norm_w * sigmoid(gate).  S [2 slots, H, dim, vdim], n [2 slots, H, dim],
+    m [2 slots, H]: read at the run's start (zeros at position 0), the run's last state written to
+    the other half."""
+    T = out.shape[0]
+    if T == 0:
+        return
+    H, dim, vdim = S.shape[1], S.shape[2], S.shape[3]
+    slots = S.shape[0] // 2
+    qf = q.float().reshape(T, H, dim) * q_scale
+    kf = k.float().reshape(T, H, dim)
+    vf = v.float().reshape(T, H, vdim)
+    g = cap * torch.tanh((z.float() + zbias.float()) / cap)
+    li, lf = g[:, :H], torch.nn.functional.logsigmoid(g[:, H:])
+    o = torch.zeros(T, H, vdim)
+    cs = cn = cm = None
+    for t in range(T):
+        code, i, f, p = int(row_state[t]), int(row_back[t]), int(row_fwd[t]), int(positions[t])
+        rd, wr = _state_rows(code, slots) if code >= 0 else (0, 0)
+        if i == 0:
+            if p > 0 and code >= 0:
+                cs, cn, cm = S[rd].clone(), n[rd].clone(), m[rd].clone()
+            else:
+                cs, cn, cm = torch.zeros(H, dim, vdim), torch.zeros(H, dim), torch.zeros(H)
+        mn = torch.maximum(lf[t] + cm, li[t])
+        a, b = torch.exp(lf[t] + cm - mn), torch.exp(li[t] - mn)
+        cs = a[:, None, None] * cs + b[:, None, None] * kf[t][:, :, None] * vf[t][:, None, :]
+        cn = a[:, None] * cn + b[:, None] * kf[t]
+        cm = mn
+        den = torch.maximum((cn * qf[t]).sum(-1).abs(), torch.exp(-cm)) + 1e-6
+        o[t] = torch.einsum("hkv,hk->hv", cs, qf[t]) / den[:, None]
+        if f == 0 and code >= 0:
+            S[wr], n[wr], m[wr] = cs, cn, cm
+    y = _rms(o, eps) * norm_w.float().view(H, vdim) * torch.sigmoid(gate.float().reshape(T, H, vdim))
+    out.copy_(y.reshape(T, H * vdim).to(out.dtype))
