@@ -48,8 +48,9 @@ __device__ __forceinline__ void ld_cols(const T* p, float* f) {
 }  // namespace
 
 // LDS (floats): qs[2][dim] | ks[2][dim] | ns[dim] | red[2][R VW] | den[2][4] | scratch[16]
-template <typename T, int CW, int NA>
-__global__ __launch_bounds__(kThreads) void mlstm_step_kernel(const MlstmArgs a, int VW, int R) {
+// NQ: key channels per thread while q and k are loaded (dim <= NQ * 256)
+template <typename T, int CW, int NA, int NQ>
+__global__ __launch_bounds__(kThreads, NA <= 4 ? 5 : NA <= 8 ? 4 : 2) void mlstm_step_kernel(const MlstmArgs a, int VW, int R) {
   const int t0 = a.run_rows != nullptr ? a.run_rows[blockIdx.x] : (int)blockIdx.x;
   const int h = blockIdx.y;
   if (t0 < 0 || a.row_back[t0] != 0) return;
@@ -88,10 +89,10 @@ __global__ __launch_bounds__(kThreads) void mlstm_step_kernel(const MlstmArgs a,
   const T* qp = static_cast<const T*>(a.q) + h * dim;
   const T* kp = static_cast<const T*>(a.k) + h * dim;
   const T* vp = static_cast<const T*>(a.v) + h * vdim + (live ? col : 0);
-  float nq[kMaxDim / kThreads], nk[kMaxDim / kThreads], nv[CW], nzi, nzf;
+  float nq[NQ], nk[NQ], nv[CW], nzi, nzf;
   auto load = [&](int64_t t) {
 #pragma unroll
-    for (int x = 0; x < kMaxDim / kThreads; ++x) {
+    for (int x = 0; x < NQ; ++x) {
       const int i = tid + x * kThreads;
       if (i < dim) {
         nq[x] = ldf(qp + t * a.qs + i);
@@ -108,7 +109,7 @@ __global__ __launch_bounds__(kThreads) void mlstm_step_kernel(const MlstmArgs a,
   for (int x = 0; x < n; ++x) {
     const int b = x & 1;
 #pragma unroll
-    for (int y = 0; y < kMaxDim / kThreads; ++y) {
+    for (int y = 0; y < NQ; ++y) {
       const int i = tid + y * kThreads;
       if (i < dim) {
         qs[b * dim + i] = nq[y] * a.q_scale;
@@ -281,8 +282,15 @@ void launch_mlstm(bool f32, const MlstmArgs& a, hipStream_t s) {
   const StepPlan p = plan_step(a.dim, a.vdim, mlstm_vec(f32, a));
   const size_t lds = step_lds(a.dim, p);
   const dim3 grid(a.run_rows != nullptr ? a.runs : a.T, a.H, p.blocks);
-#define MLSTM_GO(TT, CW, NA)                                                                   \
-  hipLaunchKernelGGL((mlstm_step_kernel<TT, CW, NA>), grid, dim3(kThreads), lds, s, a, p.VW, p.R)
+#define MLSTM_GO(TT, CW, NA)                                                                      \
+  do {                                                                                            \
+    if (a.dim <= kThreads)                                                                        \
+      hipLaunchKernelGGL((mlstm_step_kernel<TT, CW, NA, 1>), grid, dim3(kThreads), lds, s, a,     \
+                         p.VW, p.R);                                                              \
+    else                                                                                          \
+      hipLaunchKernelGGL((mlstm_step_kernel<TT, CW, NA, kMaxDim / kThreads>), grid, dim3(kThreads), \
+                         lds, s, a, p.VW, p.R);                                                   \
+  } while (0)
 #define MLSTM_NA(TT, CW)                     \
   do {                                       \
     if (p.NA <= 2) MLSTM_GO(TT, CW, 2);      \

@@ -3,8 +3,9 @@ framework at equal layer sizes: ``bench.py --arch-compare livisun`` (beside Llam
 ``--arch-compare numalorn`` (beside the Mixtral-style sparse decoder: same width, head count,
 experts, choices per token and expert width), ``--arch-compare bilolix`` (beside Numalorn:
 same width, head count, experts and expert width; attention and recurrent layers alternate
-in both) and ``--arch-compare nutitar`` (beside Bilolix with attention in every layer: same
-width, head counts and dense feed-forward width).
+in both), ``--arch-compare nutitar`` (beside Bilolix with attention in every layer: same
+width, head counts and dense feed-forward width) and ``--arch-compare modepel`` (beside Bilolix:
+attention and recurrent layers alternate in both, the same experts in every layer).
 
 Both run through the same engine (scheduler, paged cache, hipGraph decode steps), with
 random weights, a few layers of a real model's shape and a small vocabulary, so the numbers
@@ -102,6 +103,29 @@ def _nutitar_configs(name, d, H, G, F):
     return bil, nut
 
 
+def _modepel_configs(name, d, H, G, E, top, F):
+    """Bilolix and Modepel at equal sizes.  Bilolix: attention (two 64-wide maps per head, 128-wide
+    values; no window here) alternating with gla layers of d/128 heads with 64 x 128 states.
+    Modepel: attention with 128-wide heads alternating with mlstm layers of the same states.  The
+    same experts in every layer: Modepel chooses one and a half times as many among E experts and
+    E / 2 identity experts (in four groups of which three are kept), so that a token meets as many
+    computing experts on average; no shared expert (Bilolix has none)."""
+    from ..models.config import bilolix_layers, modepel_layers
+
+    bil = LayeredConfig(f"cmp-bilolix-{name}", architecture="Bilolix", vocab_size=VOCAB, hidden=d,
+                        canon_taps=0, decay_rank=64, gate_rank=64, loop=(0, 0, 1),
+                        layers=bilolix_layers("agag"[:LAYERS], H, G, 64, 128, 0, experts=E, top=top,
+                                              expert_ff=F, window=0, rot_dims=64, rot_base=5e5,
+                                              rec_heads=d // 128, rec_dim=64, moe_every=1))
+    mod = LayeredConfig(f"cmp-modepel-{name}", architecture="Modepel", vocab_size=VOCAB, hidden=d,
+                        canon_taps=0, rms_eps=1e-6,
+                        layers=modepel_layers("amam"[:LAYERS], H, G, 128, 128, 0, experts=E,
+                                              top=top + top // 2, expert_ff=F, identity=E // 2, groups=4,
+                                              keep=3, router_scale=1.5, rot_dims=64, rot_base=5e5,
+                                              rec_heads=d // 128, rec_dim=64, rec_vdim=128, moe_from=0))
+    return bil, mod
+
+
 def _engine(mcfg, args, batch):
     from ..models import layered_model_class
     from ..models.llama import DecoderLM
@@ -121,6 +145,15 @@ def _engine(mcfg, args, batch):
         from ..models.weights import init_nutitar_weights
 
         w = init_nutitar_weights(mcfg, dev, torch.bfloat16, args.seed, keep_full=False)
+        model = layered_model_class(mcfg.architecture)(mcfg, dev, weights=w)
+    elif isinstance(mcfg, LayeredConfig) and mcfg.architecture == "Modepel":
+        from ..models.weights import init_modepel_weights
+
+        w = init_modepel_weights(mcfg, dev, torch.bfloat16, args.seed, keep_full=False)
+        for lw in w["layers"]:
+            # choices spread over all outputs, as a trained correction keeps them
+            if "correction" in lw:
+                lw["correction"].mul_(0.05)
         model = layered_model_class(mcfg.architecture)(mcfg, dev, weights=w)
     elif isinstance(mcfg, LayeredConfig):
         model = layered_model_class(mcfg.architecture)(mcfg, dev, seed=args.seed)
@@ -162,9 +195,10 @@ def run(args) -> dict:
            "decode": [64, 128], "sizes": {}}
     only = [x for x in getattr(args, "arch_sizes", "").split(",") if x]
     arch = getattr(args, "arch_compare", "livisun")
-    base = {"livisun": "llama", "numalorn": "sparse", "bilolix": "numalorn", "nutitar": "bilolix"}[arch]
+    base = {"livisun": "llama", "numalorn": "sparse", "bilolix": "numalorn", "nutitar": "bilolix",
+            "modepel": "bilolix"}[arch]
     make = {"livisun": _configs, "numalorn": _moe_configs, "bilolix": _bilolix_configs,
-            "nutitar": _nutitar_configs}[arch]
+            "nutitar": _nutitar_configs, "modepel": _modepel_configs}[arch]
     for size in (SIZES if arch in ("livisun", "nutitar") else MOE_SIZES):
         name = size[0]
         if only and name not in only:

@@ -414,3 +414,126 @@ def run_nutitar(args) -> dict:
         _attention(32, 512, lens, q_lens, like, name, mfma=True)
         res[key] = {"nutitar": mine, "bilolix": like, "rows": T}
     return res
+
+
+# ---------------------------------------------------------------------------
+# Modepel's kernels (``bench.py --arch-compare modepel``) beside the like kernels of Bilolix,
+# Nutitar and Numalorn in the same run: 4096-wide layers, 32 heads over 8 key/value heads of 128,
+# 32 recurrent heads with 64 x 128 states, 8 experts and 4 identity experts.
+def _m_rows(T, d, out):
+    g = torch.Generator(device=DEV).manual_seed(0)
+    x = torch.randn(T, d, generator=g, device=DEV)
+    y = torch.randn(T, d, generator=g, device=DEV).bfloat16()
+    y2 = torch.randn(T, d, generator=g, device=DEV).bfloat16()
+    h = torch.randn(T, d, generator=g, device=DEV).bfloat16()
+    z = torch.randn(T, 13, generator=g, device=DEV) * 2
+    wt = torch.rand(T, generator=g, device=DEV)
+    out["gain_sandwich"] = _entry(_time(lambda: ops.gain_sandwich(x, y, 0.9, 1.1, 1e-6, h)), T * d * 12, 0)
+    out["gain_sandwich (shared expert, identity share)"] = _entry(
+        _time(lambda: ops.gain_sandwich(x, y, 0.9, 1.1, 1e-6, h, y2, z[:, 12], h, wt)), T * d * 16, 0)
+    F = 14336
+    u = torch.randn(T, F, generator=g, device=DEV).bfloat16()
+    o = torch.empty_like(u)
+    out["poly_norm_rows"] = _entry(_time(lambda: ops.poly_norm_rows(u, (0.4, 0.3, 0.5, 0.2), 1e-6, o)), T * F * 4, 0)
+    corr = torch.randn(12, generator=g, device=DEV) * 0.05
+    ids = torch.empty(T, 3, dtype=torch.int32, device=DEV)
+    wts = torch.empty(T, 3, device=DEV)
+    out["moe_route_softmax"] = _entry(
+        _time(lambda: ops.moe_route_softmax(z, corr, 8, 3, 4, 3, 1.5, ids, wts, wt)), T * (13 * 4 + 28), 0)
+
+
+def _m_attention(H, G, dim, lens, q_lens, out, name):
+    g = torch.Generator(device=DEV).manual_seed(3)
+    T = sum(q_lens)
+    kc, vc, pos, sl, meta = _pages(lens, q_lens, G, dim, dim, g)
+    n = (H + 2 * G) * dim
+    pr = (torch.randn(T, n + H * dim, generator=g, device=DEV) * 0.5).bfloat16()
+    pb = torch.randn(n, generator=g, device=DEV)
+    first = torch.randn(T, G * dim, generator=g, device=DEV)
+    inv, mult = ops.rotary_scaled_freq(64, 5e5, (), DEV)
+    q = torch.empty(T, H, dim, device=DEV)
+    t = _time(lambda: ops.qk_norm_rotary_append(pr, pb, None, None, False, 0, 1e-6, pos, inv, mult, 0, 0, sl, kc,
+                                                vc, H, G, dim, dim, dim, 0, q, first, 0.4, None))
+    out[f"qk_norm_rotary_append blend ({name})"] = _entry(
+        t, T * n * 2 + T * H * dim * 4 + T * G * dim * (4 + 4), 0)
+    o = torch.empty(T, H * dim, dtype=torch.bfloat16, device=DEV)
+    zero = torch.zeros(H, device=DEV)
+    pairs = sum(p + 1 for n_, q_ in zip(lens, q_lens) for p in range(n_ - q_, n_))
+    nbytes = sum(lens) * G * dim * 4 + T * H * dim * (4 + 2 + 2)
+    bt, qs, ql, kl, ws, wq = meta
+    short = ops.TALK_DECODE_MAX_ROWS if name == "decode" else 0
+    t = _time(lambda: ops.attn_keep_window(q, kc, vc, dim, bt, qs, ql, kl, ws, wq, zero, pr[:, n:], o,
+                                           dim ** -0.5, short_rows=short), reps=5, warm=2)
+    out[f"attn_keep_window unit sink, gate per output ({name})"] = _entry(t, nbytes, 4.0 * dim * H * pairs)
+
+
+def _m_memory(T, H, dim, vdim, rows, out, decode):
+    g = torch.Generator(device=DEV).manual_seed(1)
+    run = torch.nonzero(rows[1] == 0)[:, 0].to(torch.int32)
+    seqs = int(run.numel())
+    a, b, c = H * dim, 2 * H * dim, 2 * H * dim + H * vdim
+    pr = (torch.randn(T, c + H * vdim, generator=g, device=DEV) * 0.5).bfloat16()
+    z = torch.randn(T, 2 * H, generator=g, device=DEV)
+    zb = torch.randn(2 * H, generator=g, device=DEV) + 2
+    nw = torch.ones(H * vdim, device=DEV)
+    S = torch.zeros(128, H, dim, vdim, device=DEV)
+    n, m = torch.zeros(128, H, dim, device=DEV), torch.zeros(128, H, device=DEV)
+    y = torch.empty(T, H * vdim, dtype=torch.bfloat16, device=DEV)
+    nbytes = T * H * (2 * dim * 2 + vdim * 6 + 8) + (2 if decode else 1) * seqs * H * (dim * vdim + dim) * 4
+
+    def go(chunked=None):
+        return ops.mlstm_recurrence(pr[:, :a], pr[:, a:b], pr[:, b:c], z, zb, 15.0, dim ** -0.5, pr[:, c:], nw,
+                                    1e-6, S, n, m, *rows, y, run, chunked)
+
+    out["mlstm_recurrence"] = _entry(_time(go, reps=5, warm=2), nbytes, 6.0 * T * H * dim * vdim)
+    if not decode:
+        out["mlstm_recurrence (token by token)"] = _entry(_time(lambda: go(False), reps=3, warm=1), nbytes,
+                                                          6.0 * T * H * dim * vdim)
+
+
+def _m_experts(T, d, F, E, same, top, out):
+    from ..models.moe import MoEBuffers, grouped_ok, moe_mlp
+
+    g = torch.Generator(device=DEV).manual_seed(3)
+    h = torch.randn(T, d, generator=g, device=DEV).bfloat16()
+    w13 = (torch.randn(E, 2 * F, d, generator=g, device=DEV) * d ** -0.5).bfloat16()
+    w2 = (torch.randn(E, d, F, generator=g, device=DEV) * F ** -0.5).bfloat16()
+    z = torch.randn(T, E + same, generator=g, device=DEV) * 2
+    corr = torch.randn(E + same, generator=g, device=DEV) * 0.05
+    ident = torch.empty(T, device=DEV)
+    if not grouped_ok(w13, w2):
+        return
+    bufs = MoEBuffers.allocate(T, top, E + 1, d, F, DEV, torch.bfloat16)
+    dummy = z.new_zeros(E, d)
+    t = _time(lambda: moe_mlp(h, dummy, w13, w2, top, bufs, spare=True,
+                              routing=lambda w, i: ops.moe_route_softmax(z, corr, E, top, 4, 3, 1.5, i, w, ident)),
+              reps=10, warm=2)
+    real = int((bufs.ids[:T] < E).sum())
+    used = int(torch.unique(bufs.ids[:T][bufs.ids[:T] < E]).numel())
+    out["experts (route + grouped GEMMs + combine)"] = _entry(
+        t, used * 3 * d * F * 2 + T * d * 4, 6.0 * real * d * F)
+
+
+def run_modepel(args) -> dict:
+    torch.manual_seed(0)
+    d, H, G, dim, RH, rd, rv = 4096, 32, 8, 128, 32, 64, 128
+    res = {"width": d, "heads": [H, G], "head": dim, "recurrent_heads": [RH, rd, rv], "experts": [8, 4, 3, 14336]}
+    for name, lens, q_lens, key in (("prefill", [2048, 600], [2048, 600], "prefill_step_4096_rows"),
+                                    ("decode", [600] * 64, [1] * 64, "decode_step_64_rows")):
+        mine, like = {}, {}
+        pre = name == "prefill"
+        rl, sl, first = ([2048, 2048], [0, 63], 0) if pre else ([1] * 64, list(range(64)), 600)
+        T = sum(rl)
+        _m_rows(T, d, mine)
+        _m_attention(H, G, dim, lens, q_lens, mine, name)
+        rows = _runs(rl, sl, first)
+        _m_memory(T, RH, rd, rv, rows, mine, not pre)
+        _m_experts(T, d, 14336, 8, 4, 3, mine)
+        _b_rows(T, d, like)
+        _n_rows(T, d, rl, sl, like, first)
+        _n_attention("window", H, G, lens, q_lens, like, name, 4096, 0)
+        _n_attention("keyval", H, G, lens, q_lens, like, name)
+        _b_recurrence(T, RH, rd, rv, rows, like, not pre)
+        _experts(T, d, 14336, 8, 2, like)
+        res[key] = {"modepel": mine, "like": like}
+    return res

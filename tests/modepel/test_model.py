@@ -336,7 +336,7 @@ def test_mfma_sized_model_in_bf16_against_fp32():
     got = run_schedule(eng, steps)
     assert len(got) == len(want) == 48
     e = sorted(spread(row, want[k], want[k].double().std()) for k, row in got.items())
-    assert e[len(e) // 2] < 0.03 and e[-5] < 0.15, e[-8:]
+    assert e[len(e) // 2] < 0.05 and e[-5] < 0.15, e[-8:]
 
 
 @pytest.mark.gpu
