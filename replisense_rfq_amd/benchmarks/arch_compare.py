@@ -103,26 +103,32 @@ def _nutitar_configs(name, d, H, G, F):
     return bil, nut
 
 
-def _modepel_configs(name, d, H, G, E, top, F):
+def _modepel_configs(name, d, H, G, *ff):
     """Bilolix and Modepel at equal sizes.  Bilolix: attention (two 64-wide maps per head, 128-wide
     values; no window here) alternating with gla layers of d/128 heads with 64 x 128 states.
     Modepel: attention with 128-wide heads alternating with mlstm layers of the same states.  The
     same experts in every layer: Modepel chooses one and a half times as many among E experts and
-    E / 2 identity experts (in four groups of which three are kept), so that a token meets as many
-    computing experts on average; no shared expert (Bilolix has none)."""
+    E / 2 identity experts (in six groups of which four are kept), so that a token meets as many
+    computing experts on average; no shared expert (Bilolix has none).  ff: (width,) for dense
+    feed-forwards in both, (experts, choices, width) for mixtures."""
     from ..models.config import bilolix_layers, modepel_layers
+
+    if len(ff) == 1:
+        b_ff, m_ff = dict(ff=ff[0]), dict(ff=ff[0])
+    else:
+        E, top, F = ff
+        b_ff = dict(ff=0, experts=E, top=top, expert_ff=F, moe_every=1)
+        m_ff = dict(ff=0, experts=E, top=top + top // 2, expert_ff=F, identity=E // 2, groups=6, keep=4,
+                    router_scale=1.2, moe_from=0)
 
     bil = LayeredConfig(f"cmp-bilolix-{name}", architecture="Bilolix", vocab_size=VOCAB, hidden=d,
                         canon_taps=0, decay_rank=64, gate_rank=64, loop=(0, 0, 1),
-                        layers=bilolix_layers("agag"[:LAYERS], H, G, 64, 128, 0, experts=E, top=top,
-                                              expert_ff=F, window=0, rot_dims=64, rot_base=5e5,
-                                              rec_heads=d // 128, rec_dim=64, moe_every=1))
+                        layers=bilolix_layers("agag"[:LAYERS], H, G, 64, 128, window=0, rot_dims=64,
+                                              rot_base=5e5, rec_heads=d // 128, rec_dim=64, **b_ff))
     mod = LayeredConfig(f"cmp-modepel-{name}", architecture="Modepel", vocab_size=VOCAB, hidden=d,
                         canon_taps=0, rms_eps=1e-6,
-                        layers=modepel_layers("amam"[:LAYERS], H, G, 128, 128, 0, experts=E,
-                                              top=top + top // 2, expert_ff=F, identity=E // 2, groups=4,
-                                              keep=3, router_scale=1.5, rot_dims=64, rot_base=5e5,
-                                              rec_heads=d // 128, rec_dim=64, rec_vdim=128, moe_from=0))
+                        layers=modepel_layers("amam"[:LAYERS], H, G, 128, 128, rot_dims=64, rot_base=5e5,
+                                              rec_heads=d // 128, rec_dim=64, rec_vdim=128, **m_ff))
     return bil, mod
 
 
@@ -199,7 +205,9 @@ def run(args) -> dict:
             "modepel": "bilolix"}[arch]
     make = {"livisun": _configs, "numalorn": _moe_configs, "bilolix": _bilolix_configs,
             "nutitar": _nutitar_configs, "modepel": _modepel_configs}[arch]
-    for size in (SIZES if arch in ("livisun", "nutitar") else MOE_SIZES):
+    sizes = SIZES[:2] + MOE_SIZES if arch == "modepel" else \
+        SIZES if arch in ("livisun", "nutitar") else MOE_SIZES
+    for size in sizes:
         name = size[0]
         if only and name not in only:
             continue

@@ -439,7 +439,7 @@ def _m_rows(T, d, out):
     ids = torch.empty(T, 3, dtype=torch.int32, device=DEV)
     wts = torch.empty(T, 3, device=DEV)
     out["moe_route_softmax"] = _entry(
-        _time(lambda: ops.moe_route_softmax(z, corr, 8, 3, 4, 3, 1.5, ids, wts, wt)), T * (13 * 4 + 28), 0)
+        _time(lambda: ops.moe_route_softmax(z, corr, 8, 3, 6, 4, 1.2, ids, wts, wt)), T * (13 * 4 + 28), 0)
 
 
 def _m_attention(H, G, dim, lens, q_lens, out, name):
@@ -506,7 +506,7 @@ def _m_experts(T, d, F, E, same, top, out):
     bufs = MoEBuffers.allocate(T, top, E + 1, d, F, DEV, torch.bfloat16)
     dummy = z.new_zeros(E, d)
     t = _time(lambda: moe_mlp(h, dummy, w13, w2, top, bufs, spare=True,
-                              routing=lambda w, i: ops.moe_route_softmax(z, corr, E, top, 4, 3, 1.5, i, w, ident)),
+                              routing=lambda w, i: ops.moe_route_softmax(z, corr, E, top, 6, 4, 1.2, i, w, ident)),
               reps=10, warm=2)
     real = int((bufs.ids[:T] < E).sum())
     used = int(torch.unique(bufs.ids[:T][bufs.ids[:T] < E]).numel())

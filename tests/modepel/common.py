@@ -63,7 +63,7 @@ ODD = config([attn(3, 3, 6, 10, 6, dense(18)), memory(3, 7, 9, moe(5, 2, 11, ide
              vocab=53, width=37)
 # sizes the MFMA tiles cover (bf16 on the GPU); sixteen heads over one key head: decoded rows take
 # the heads-as-columns form
-WIDE = config([attn(8, 2, 32, 32, 16, dense(64), scale=0.2), memory(2, 32, 48, moe(4, 2, 32, identity=2, shared=32)),
+WIDE = config([attn(8, 2, 32, 32, 16, dense(64), scale=0.2), memory(3, 32, 80, moe(4, 2, 32, identity=2, shared=32)),
                attn(16, 2, 64, 32, 32, moe(4, 2, 32), scale=0.15), attn(16, 1, 32, 64, 16, None, v_mix=False),
                memory(1, 64, 80, dense(64))],
               width=64, vocab=90)
