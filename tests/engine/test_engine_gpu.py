@@ -254,6 +254,7 @@ def test_chunked_prefill_steps_without_logits(gpu, monkeypatch):
     previous step's upload could read the next payload).  Every step is checked to have
     finished before the next upload, and the documents must decode to valid JSON twice
     over with identical tokens."""
+    from replisense_rfq_amd import ops
     from replisense_rfq_amd.engine import runner as runner_mod
 
     waits = []
@@ -266,10 +267,14 @@ def test_chunked_prefill_steps_without_logits(gpu, monkeypatch):
 
     monkeypatch.setattr(runner_mod.ModelRunner, "_run", _run)
     texts = []
+    ops.reset_plans()              # an earlier engine's start-up plans do not fit an untuned one
     for _ in range(2):
         eng = LLMEngine(EngineConfig(model="tiny-llama", max_num_seqs=4, max_kv_blocks=2048,
                                      max_batched_tokens=96, graph_buckets=(1, 2, 4),
-                                     decode_hints=True))
+                                     decode_hints=True,
+                                     # plans chosen by timing may differ between the engines
+                                     # and round differently: a near tie then flips a token
+                                     tune_gemm=False))
         tok = eng.tokenizer
         prompts = [tok.chat_ids(build_messages(synth.make_long_rfq(i).text)) for i in range(2)]
         assert all(len(p) > 3 * 96 for p in prompts)
