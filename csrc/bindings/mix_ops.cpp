@@ -74,21 +74,30 @@ bool launch_qk_norm_rotary_append(bool, const void*, int64_t, const float*, cons
                                   const float*, bool, int, float, const int32_t*, const float*, int,
                                   float, int, int, const int32_t*, void*, void*, int, int, int, int,
                                   int, int, int, int, int64_t, const float*, float, float*, float*,
-                                  hipStream_t);
+                                  bool, const float*, int, float*, int, const int32_t*,
+                                  const int32_t*, const int32_t*, hipStream_t);
 bool launch_attn_keep_window(bool, const float*, const void*, const void*, int64_t, const int32_t*,
                              int, const int32_t*, const int32_t*, const int32_t*, const int32_t*,
                              const int32_t*, int, const float*, const void*, int64_t, int, void*,
-                             int64_t, float, int, int, bool, int, int, int, int, int, hipStream_t);
+                             int64_t, float, int, int, bool, int, int, int, int, int, float, float,
+                             hipStream_t);
 int launch_attn_keep_decode(bool, const float*, const void*, const void*, int64_t, const int32_t*,
                             int, const int32_t*, const int32_t*, const int32_t*, int, int,
                             const float*, const void*, int64_t, int, void*, int64_t, float, int,
-                            int, bool, int, int, int, int, int, hipStream_t);
+                            int, bool, int, int, int, int, int, float, float, hipStream_t);
 bool keep_mfma_ok(int, int, int, bool);
 bool launch_attn_keep_mfma(const float*, const void*, const void*, int64_t, const int32_t*, int,
                            const int32_t*, const int32_t*, const int32_t*, const int32_t*,
                            const int32_t*, int, const float*, const void*, int64_t, int, void*,
                            int64_t, float, int, int, bool, int, int, int, int, int, bool, int, int,
-                           hipStream_t);
+                           float, float, hipStream_t);
+bool streams_norm_ok(int, int64_t);
+void launch_streams_norm(bool, float*, const int32_t*, const void*, int, const void*, int64_t,
+                         const float*, const float*, const float*, const float*, float, bool, void*,
+                         int, int, int, bool, hipStream_t);
+void launch_gelu_glu_rows(bool, const void*, int64_t, void*, int64_t, int, int, hipStream_t);
+void launch_gate_heads(bool, const void*, int64_t, int64_t, const void*, int64_t, void*, int64_t, int,
+                       int, int, hipStream_t);
 void launch_gain_sandwich(bool, float*, const void*, int64_t, bool, const void*, int64_t, bool,
                           const float*, int64_t, const void*, int64_t, bool, const float*, float,
                           float, float, void*, int, int, hipStream_t);
@@ -665,7 +674,9 @@ void qk_norm_rotary_append(const Tensor& proj, const OptT& bias, const OptT& q_n
                            const OptT& k_cache, const OptT& v_cache, int64_t H, int64_t G,
                            int64_t qw, int64_t kw, int64_t vdim, int64_t v_mode,
                            const Tensor& q_out, const OptT& v_in, double v_take,
-                           const OptT& v_out) {
+                           const OptT& v_out, bool neighbours, const OptT& conv_w,
+                           const OptT& conv_state, const OptT& row_state, const OptT& row_back,
+                           const OptT& row_fwd) {
   const bool f32 = act_f32(proj, "qk_norm_rotary_append proj");
   TORCH_CHECK(proj.dim() == 2 && proj.stride(1) == 1, "qk_norm_rotary_append: proj [T, N]");
   const int T = (int)proj.size(0);
@@ -708,6 +719,23 @@ void qk_norm_rotary_append(const Tensor& proj, const OptT& bias, const OptT& q_n
   TORCH_CHECK((!v_in.has_value() && !v_out.has_value()) || (v_mode != 2 && G > 0),
               "qk_norm_rotary_append: blended values need values");
   const int64_t nv = (int64_t)T * G * vdim;
+  int taps = 0, state_slots = 0;
+  float* cst = nullptr;
+  const int32_t *rs = nullptr, *rb = nullptr, *rf = nullptr;
+  if (conv_w.has_value()) {
+    TORCH_CHECK(conv_w->dim() == 2 && conv_w->size(0) >= 1 && conv_w->size(1) == W && !bias.has_value() &&
+                conv_state.has_value() && conv_state->dim() == 3 && conv_state->size(0) % 2 == 0 &&
+                conv_state->size(1) == conv_w->size(0) - 1 && conv_state->size(2) == W &&
+                row_state.has_value() && row_back.has_value() && row_fwd.has_value(),
+                "qk_norm_rotary_append: conv_w [taps, row width] without bias, conv_state "
+                "[2S, taps-1, row width] and the rows' places");
+    taps = (int)conv_w->size(0);
+    state_slots = (int)conv_state->size(0) / 2;
+    cst = const_cast<float*>(f32p(*conv_state, "conv_state"));
+    rs = i32p(*row_state, "row_state", T);
+    rb = i32p(*row_back, "row_back", T);
+    rf = i32p(*row_fwd, "row_fwd", T);
+  }
   const float* fr = nrot > 0 ? f32p(inv_freq, "inv_freq") : nullptr;
   const bool ok = rfqmix::launch_qk_norm_rotary_append(
       f32, proj.data_ptr(), proj.stride(0), optf(bias, "bias", W), optf(q_norm_w, "q_norm_w", nqw),
@@ -716,6 +744,7 @@ void qk_norm_rotary_append(const Tensor& proj, const OptT& bias, const OptT& q_n
       (int)q_rot_off, (int)k_rot_off, i32p(slots, "slots", T), kp, vp, T, (int)H, (int)G, (int)qw,
       (int)kw, (int)vdim, (int)v_mode, BS, pool_slots, optf(v_in, "v_in", nv), (float)v_take,
       const_cast<float*>(optf(v_out, "v_out", nv)), const_cast<float*>(f32p(q_out, "q_out")),
+      neighbours, taps > 0 ? f32p(*conv_w, "conv_w") : nullptr, taps, cst, state_slots, rs, rb, rf,
       stream());
   TORCH_CHECK(ok, "qk_norm_rotary_append: a row does not fit the LDS");
 }
@@ -725,7 +754,7 @@ void attn_keep_window(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
                       const Tensor& kv_len, const Tensor& work_seq, const Tensor& work_qblk,
                       const OptT& head_bias, const OptT& gate, const Tensor& out, double scale,
                       int64_t window, int64_t keep_first, bool sigmoid, int64_t short_rows,
-                      bool mfma) {
+                      bool mfma, double softcap, double out_mult) {
   const bool f32 = act_f32(k_cache, "attn_keep_window k_cache");
   TORCH_CHECK(q.dim() == 3, "attn_keep_window: q [T, H, E]");
   const int T = (int)q.size(0), H = (int)q.size(1), E = (int)q.size(2);
@@ -775,7 +804,8 @@ void attn_keep_window(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
         f32, f32p(q, "q"), k_cache.data_ptr(), v_cache.data_ptr(), vrs, i32p(bt, "block_tables", 0),
         (int)bt.size(1), i32p(q_start, "q_start", NB), i32p(q_len, "q_len", NB),
         i32p(kv_len, "kv_len", NB), NB, (int)short_rows, hb, gp, gs, gw, out.data_ptr(), out.stride(0),
-        (float)scale, (int)window, (int)keep_first, sigmoid, H, G, E, (int)vdim, BS, stream());
+        (float)scale, (int)window, (int)keep_first, sigmoid, H, G, E, (int)vdim, BS, (float)softcap,
+        (float)out_mult, stream());
     if (kt > 0) return;
   }
   if (tiles) {
@@ -784,7 +814,8 @@ void attn_keep_window(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
         (int)bt.size(1), i32p(q_start, "q_start", NB), i32p(q_len, "q_len", NB),
         i32p(kv_len, "kv_len", NB), i32p(work_seq, "work_seq", W), i32p(work_qblk, "work_qblk", W),
         W, hb, gp, gs, gw, out.data_ptr(), out.stride(0), (float)scale, (int)window, (int)keep_first,
-        sigmoid, H, G, E, (int)vdim, BS, shared, NB, (int)short_rows, stream());
+        sigmoid, H, G, E, (int)vdim, BS, shared, NB, (int)short_rows, (float)softcap, (float)out_mult,
+        stream());
     return;
   }
   const bool ok = rfqmix::launch_attn_keep_window(
@@ -792,7 +823,7 @@ void attn_keep_window(const Tensor& q, const Tensor& k_cache, const Tensor& v_ca
       (int)bt.size(1), i32p(q_start, "q_start", NB), i32p(q_len, "q_len", NB),
       i32p(kv_len, "kv_len", NB), i32p(work_seq, "work_seq", W), i32p(work_qblk, "work_qblk", W), W,
       hb, gp, gs, gw, out.data_ptr(), out.stride(0), (float)scale, (int)window, (int)keep_first,
-      sigmoid, H, G, E, (int)vdim, BS, stream());
+      sigmoid, H, G, E, (int)vdim, BS, (float)softcap, (float)out_mult, stream());
   TORCH_CHECK(ok, "attn_keep_window: value size too large for the LDS");
 }
 
@@ -857,8 +888,7 @@ void gated_linear_recurrence(const Tensor& q, const Tensor& k, const Tensor& v, 
               "gated_linear_recurrence: z [T, H dim] float32");
   TORCH_CHECK(gate.is_cuda() && gate.scalar_type() == out.scalar_type() &&
               rows2d(gate, T, (int64_t)H * vdim), "gated_linear_recurrence: gate [T, H vdim]");
-  TORCH_CHECK(rows2d(out, T, (int64_t)H * vdim) && out.is_contiguous(),
-              "gated_linear_recurrence: out [T, H vdim]");
+  TORCH_CHECK(rows2d(out, T, (int64_t)H * vdim), "gated_linear_recurrence: out [T, H vdim]");
   TORCH_CHECK(rfqmix::linrec_ok(dim, vdim) && H <= 65535,
               "gated_linear_recurrence: head sizes outside the kernel's range");
   rfqmix::LinrecArgs a;
@@ -883,7 +913,7 @@ void gated_linear_recurrence(const Tensor& q, const Tensor& k, const Tensor& v, 
   a.row_fwd = i32p(row_fwd, "row_fwd", T); a.pos = i32p(pos, "positions", T);
   a.run_rows = run_rows.has_value() ? i32p(*run_rows, "run_rows", 0) : nullptr;
   a.runs = run_rows.has_value() ? (int)run_rows->numel() : 0;
-  a.out = out.data_ptr();
+  a.out = out.data_ptr(); a.os = out.stride(0);
   a.T = T; a.H = H; a.rep = H / Hq; a.dim = dim; a.vdim = vdim; a.slots = (int)state.size(0) / 2;
   rfqmix::launch_gated_linrec(in_f32, a_f32, beta.has_value(), a, stream());
 }
@@ -919,6 +949,59 @@ void gelu_rows(const Tensor& x, const Tensor& out) {
               "gelu_rows: x, out [T, F] of one type");
   rfqmix::launch_gelu_rows(f32, x.data_ptr(), x.stride(0), out.data_ptr(), out.stride(0),
                            (int)x.size(0), (int)x.size(1), stream());
+}
+
+// ---- several residual streams
+void streams_norm(const Tensor& x, const OptT& y, const OptT& mix, const OptT& w_out,
+                  const Tensor& w_in, const Tensor& w, double eps, bool centre, const Tensor& out,
+                  bool keep, const OptT& ids, const OptT& table) {
+  const bool f32 = act_f32(out, "streams_norm out");
+  TORCH_CHECK(x.dim() == 3, "streams_norm: x [T, S, d]");
+  const int T = (int)x.size(0), S = (int)x.size(1), d = (int)x.size(2);
+  TORCH_CHECK(rfqmix::streams_norm_ok(S, d), "streams_norm: at most 16 streams, the row fits the LDS");
+  TORCH_CHECK(rows2d(out, T, d) && out.is_contiguous(), "streams_norm: out [T, d]");
+  const void *yp = nullptr, *tp = nullptr;
+  int64_t ys = 0;
+  int vocab = 0;
+  if (y.has_value()) {
+    TORCH_CHECK(y->is_cuda() && y->scalar_type() == out.scalar_type() && rows2d(*y, T, d) &&
+                mix.has_value() && w_out.has_value(), "streams_norm: y [T, d] with its weights");
+    yp = y->data_ptr();
+    ys = y->stride(0);
+  }
+  if (ids.has_value()) {
+    TORCH_CHECK(table.has_value() && table->is_cuda() && table->scalar_type() == out.scalar_type() &&
+                table->is_contiguous() && table->dim() == 2 && table->size(0) >= 1 && table->size(1) == d,
+                "streams_norm: table [V, d]");
+    tp = table->data_ptr();
+    vocab = (int)table->size(0);
+  }
+  rfqmix::launch_streams_norm(
+      f32, const_cast<float*>(f32p(x, "x")), ids.has_value() ? i32p(*ids, "ids", T) : nullptr, tp, vocab,
+      yp, ys, yp ? f32p(*mix, "mix", (int64_t)S * S) : nullptr, yp ? f32p(*w_out, "w_out", S) : nullptr,
+      f32p(w_in, "w_in", S), f32p(w, "w", d), (float)eps, centre, out.data_ptr(), T, d, S, keep, stream());
+}
+
+void gelu_glu_rows(const Tensor& gu, const Tensor& out) {
+  const bool f32 = act_f32(gu, "gelu_glu_rows gate_up");
+  TORCH_CHECK(gu.dim() == 2 && gu.stride(1) == 1 && gu.size(1) % 2 == 0 && out.is_cuda() &&
+              out.scalar_type() == gu.scalar_type() && rows2d(out, gu.size(0), gu.size(1) / 2),
+              "gelu_glu_rows: gate_up [T, 2F], out [T, F] of one type");
+  TORCH_CHECK((gu.size(1) + 511) / 512 <= 65535, "gelu_glu_rows: F too large");
+  rfqmix::launch_gelu_glu_rows(f32, gu.data_ptr(), gu.stride(0), out.data_ptr(), out.stride(0),
+                               (int)gu.size(0), (int)out.size(1), stream());
+}
+
+void gate_heads(const Tensor& x, const Tensor& gate, const Tensor& out) {
+  const bool f32 = act_f32(x, "gate_heads x");
+  TORCH_CHECK(x.dim() == 3 && x.stride(2) == 1, "gate_heads: x [H, T, n]");
+  const int64_t H = x.size(0), T = x.size(1), n = x.size(2);
+  TORCH_CHECK(H >= 1 && n >= 1 && gate.is_cuda() && gate.scalar_type() == x.scalar_type() &&
+              rows2d(gate, T, H * n) && out.is_cuda() && out.scalar_type() == x.scalar_type() &&
+              rows2d(out, T, H * n), "gate_heads: gate, out [T, H n] in the type of x");
+  TORCH_CHECK((H * n + 255) / 256 <= 65535, "gate_heads: too wide");
+  rfqmix::launch_gate_heads(f32, x.data_ptr(), x.stride(0), x.stride(1), gate.data_ptr(), gate.stride(0),
+                            out.data_ptr(), out.stride(0), (int)T, (int)H, (int)n, stream());
 }
 
 void gain_sandwich(const Tensor& x, const OptT& y, const OptT& y2, const OptT& y2_logit,
@@ -1050,6 +1133,9 @@ bool mlstm_chunk_ok(int64_t dim, int64_t vdim) {
 }  // namespace
 
 TORCH_LIBRARY(rfq_mix, m) {
+  m.def("streams_norm(Tensor(a!) x, Tensor? y, Tensor? mix, Tensor? w_out, Tensor w_in, Tensor w, float eps, bool centre, Tensor(b!) out, bool keep, Tensor? ids, Tensor? table) -> ()");
+  m.def("gelu_glu_rows(Tensor gate_up, Tensor(a!) out) -> ()");
+  m.def("gate_heads(Tensor x, Tensor gate, Tensor(a!) out) -> ()");
   m.def("gain_sandwich(Tensor(a!) x, Tensor? y, Tensor? y2, Tensor? y2_logit, Tensor? h_in, Tensor? h_weight, float g_post, float g_pre, float eps, Tensor(b!)? out) -> ()");
   m.def("poly_norm_rows(Tensor x, float a, float b, float c, float e, float eps, Tensor(a!) out) -> ()");
   m.def("moe_route_softmax(Tensor z, Tensor correction, int real, int top, int groups, int keep, float scale, Tensor(a!) ids, Tensor(b!) weights, Tensor(c!)? ident) -> ()");
@@ -1081,8 +1167,8 @@ TORCH_LIBRARY(rfq_mix, m) {
   m.def("rotary_append(Tensor qkv, Tensor pos, Tensor inv_freq, Tensor slots, Tensor(a!) k_cache, Tensor(b!) v_cache, int H, int G, int maps, int dim, int vdim, Tensor(c!) q_out) -> ()");
   m.def("attn_diff_window(Tensor q, Tensor k_cache, Tensor v_cache, Tensor bt, Tensor q_start, Tensor q_len, Tensor kv_len, Tensor work_seq, Tensor work_qblk, Tensor gate, Tensor(a!) out, float scale, int window, float lam, float eps, float out_mult, int short_rows, bool mfma) -> ()");
   m.def("diff_mfma_ok", &diff_mfma_ok);
-  m.def("qk_norm_rotary_append(Tensor proj, Tensor? bias, Tensor? q_norm_w, Tensor? k_norm_w, bool norm_all, int k_norm_n, float eps, Tensor pos, Tensor inv_freq, float rot_mult, int q_rot_off, int k_rot_off, Tensor slots, Tensor(a!)? k_cache, Tensor(b!)? v_cache, int H, int G, int qw, int kw, int vdim, int v_mode, Tensor(c!) q_out, Tensor? v_in, float v_take, Tensor(d!)? v_out) -> ()");
-  m.def("attn_keep_window(Tensor q, Tensor k_cache, Tensor v_cache, int vdim, Tensor bt, Tensor q_start, Tensor q_len, Tensor kv_len, Tensor work_seq, Tensor work_qblk, Tensor? head_bias, Tensor? gate, Tensor(a!) out, float scale, int window, int keep_first, bool sigmoid, int short_rows, bool mfma) -> ()");
+  m.def("qk_norm_rotary_append(Tensor proj, Tensor? bias, Tensor? q_norm_w, Tensor? k_norm_w, bool norm_all, int k_norm_n, float eps, Tensor pos, Tensor inv_freq, float rot_mult, int q_rot_off, int k_rot_off, Tensor slots, Tensor(a!)? k_cache, Tensor(b!)? v_cache, int H, int G, int qw, int kw, int vdim, int v_mode, Tensor(c!) q_out, Tensor? v_in, float v_take, Tensor(d!)? v_out, bool neighbours, Tensor? conv_w, Tensor(e!)? conv_state, Tensor? row_state, Tensor? row_back, Tensor? row_fwd) -> ()");
+  m.def("attn_keep_window(Tensor q, Tensor k_cache, Tensor v_cache, int vdim, Tensor bt, Tensor q_start, Tensor q_len, Tensor kv_len, Tensor work_seq, Tensor work_qblk, Tensor? head_bias, Tensor? gate, Tensor(a!) out, float scale, int window, int keep_first, bool sigmoid, int short_rows, bool mfma, float softcap, float out_mult) -> ()");
   m.def("keep_mfma_ok", &keep_mfma_ok);
   m.def("xielu_rows(Tensor x, float ap, float an, Tensor(a!) out) -> ()");
   m.def("conv_act_heads(Tensor x, Tensor w, Tensor(a!) state, Tensor row_state, Tensor row_back, Tensor row_fwd, Tensor pos, int n_unit, int dim, float unit_eps, Tensor(b!) out) -> ()");
@@ -1094,6 +1180,9 @@ TORCH_LIBRARY(rfq_mix, m) {
 }
 
 TORCH_LIBRARY_IMPL(rfq_mix, CUDA, m) {
+  m.impl("streams_norm", &streams_norm);
+  m.impl("gelu_glu_rows", &gelu_glu_rows);
+  m.impl("gate_heads", &gate_heads);
   m.impl("gain_sandwich", &gain_sandwich);
   m.impl("poly_norm_rows", &poly_norm_rows);
   m.impl("moe_route_softmax", &moe_route_softmax);

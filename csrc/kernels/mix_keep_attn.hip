@@ -2,17 +2,18 @@
 // window that keeps the first tokens, for softmax, sink-softmax and sigmoid weights.
 //
 //   qk_norm_rotary_append   rows q [H, qw] | k [G, kw] (| v [G, vdim]) of a fused projection:
-//                           bias, RMS norm per head or over the whole projection, rotation of
-//                           entries (off + i, off + i + n) by pos * f_i with a factor on cos and
-//                           sin; q out in fp32, k and the values into their page rows; the
+//                           bias, causal convolution over the sequence's rows, RMS norm per head or
+//                           over the whole projection, rotation of entries (off + i, off + i + n) or
+//                           (off + 2i, off + 2i + 1) by pos * f_i with a factor on cos and sin; q out in fp32, k and the values into their page rows; the
 //                           values may be blended with another layer's values of the same token
 //                           (v <- keep v + take v_in) and handed on unblended (v_out)
 //   attn_keep_window        s(i, j) = scale q_h(i) . k_g(j);  i sees j <= i with
-//                           i - j < window or j < keep_first (window 0: every j <= i)
+//                           i - j < window or j < keep_first (window 0: every j <= i);
+//                           softcap > 0: s <- softcap tanh(s / softcap)
 //                             softmax:  w = exp(s) / (sum_j' exp(s(i, j')) [+ exp(bias_h)])
 //                             sigmoid:  w = 1 / (1 + exp(-(s + bias_h))), not normalised
 //                           out(i) = sum_j w v_g(j) [* sigmoid(gate(i, h)) or, with a gate column
-//                           per output (gate_w = vdim), * sigmoid(gate(i, h, dv))]
+//                           per output (gate_w = vdim), * sigmoid(gate(i, h, dv))] * out_mult
 //                           The values are the first vdim entries of rows of stride vrs, so the
 //                           key pages themselves can be the values (latent attention).
 //   xielu_rows              z > 0: ap z^2 + z / 2;  z <= 0: an (exp(z) - 1 - z) + z / 2
@@ -30,6 +31,10 @@ constexpr int KQB = 32;     // queries per work item
 constexpr int KKT = 64;     // keys per tile
 constexpr int KEC = 32;     // dimensions per LDS slice
 constexpr float kNegInfK = -__builtin_huge_valf();
+
+__device__ __forceinline__ float capped(float s, float cap) {
+  return cap > 0.f ? cap * tanhf(s / cap) : s;
+}
 }  // namespace
 
 // ------------------------------------------------------------------ norm, rotation, append
@@ -87,6 +92,9 @@ __device__ __forceinline__ void st_chunk(bf16_t* p, const float* f) {
 
 // One workgroup per row; the row passes through LDS as floats.  CW = 8: every width, stride and
 // pointer is a multiple of 8 values / 16 bytes, a thread moves chunks of 8 neighbouring values.
+// conv_w [taps][W]: the row is first convolved over the rows of its sequence (rows before the run
+// come from the state half that row_state names, zeros before position 0; the run's last taps - 1
+// rows go to the other half).
 // LDS (floats): row[W] | fac[H + G] | cs[2 nrot] | scratch[16]
 template <typename T, int CW>
 __global__ __launch_bounds__(256) void qk_norm_rotary_append_kernel(
@@ -96,7 +104,10 @@ __global__ __launch_bounds__(256) void qk_norm_rotary_append_kernel(
     int nrot, float rot_mult, int q_rot_off, int k_rot_off, const int32_t* __restrict__ slots,
     T* __restrict__ k_cache, T* __restrict__ v_cache, int H, int G, int qw, int kw, int vdim,
     int v_mode, int BS, int64_t pool_slots, const float* __restrict__ v_in, float v_keep,
-    float v_take, float* __restrict__ v_out, float* __restrict__ q_out) {
+    float v_take, float* __restrict__ v_out, float* __restrict__ q_out, int neighbours,
+    const float* __restrict__ conv_w, int taps, float* __restrict__ conv_state, int state_slots,
+    const int32_t* __restrict__ row_state, const int32_t* __restrict__ row_back,
+    const int32_t* __restrict__ row_fwd) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int t = blockIdx.x, tid = threadIdx.x, nthr = blockDim.x;
   const int lane = tid & 63, wid = tid >> 6, nw = nthr >> 6;
@@ -110,9 +121,45 @@ __global__ __launch_bounds__(256) void qk_norm_rotary_append_kernel(
   // the row into LDS; with whole-projection norms the squares are summed on the way
   const T* src = proj + (int64_t)t * stride;
   float sq = 0.f, sk = 0.f;
+  const int K = taps - 1;              // taps > 0 with a convolution
+  int back = 0, fwd = 0, pt = 0;
+  const float* rd = nullptr;
+  float* wr = nullptr;
+  if (conv_w != nullptr) {
+    const int code = row_state[t];
+    back = row_back[t];
+    fwd = row_fwd[t];
+    pt = pos[t];
+    if (code >= 0) {
+      rd = conv_state + ((int64_t)((code & 1) * state_slots + (code >> 1)) * K) * W;
+      wr = conv_state + ((int64_t)((1 - (code & 1)) * state_slots + (code >> 1)) * K) * W;
+    }
+  }
   for (int c = tid * CW; c < W; c += nthr * CW) {
     float f[CW];
     ld_chunk<CW>(src + c, f);
+    if (conv_w != nullptr) {
+      float u[CW], w[CW];
+      if (wr != nullptr) {
+        if (fwd < K) st_chunk<CW>(wr + (int64_t)(K - 1 - fwd) * W + c, f);
+        if (back == 0)                 // a run shorter than the taps: older inputs move up
+          for (int e = 0; e < K - (fwd + 1); ++e) {
+            ld_chunk<CW>(rd + (int64_t)(e + fwd + 1) * W + c, u);
+            st_chunk<CW>(wr + (int64_t)e * W + c, u);
+          }
+      }
+      ld_chunk<CW>(conv_w + (int64_t)K * W + c, w);
+#pragma unroll
+      for (int i = 0; i < CW; ++i) f[i] *= w[i];
+      for (int dl = 1; dl <= K; ++dl) {
+        if (dl <= back) ld_chunk<CW>(src - (int64_t)dl * stride + c, u);
+        else if (pt - dl >= 0 && rd != nullptr) ld_chunk<CW>(rd + (int64_t)(K + back - dl) * W + c, u);
+        else break;
+        ld_chunk<CW>(conv_w + (int64_t)(K - dl) * W + c, w);
+#pragma unroll
+        for (int i = 0; i < CW; ++i) f[i] += w[i] * u[i];
+      }
+    }
     if (bias != nullptr) {
       float b[CW];
       ld_chunk<CW>(bias + c, b);
@@ -219,7 +266,16 @@ __global__ __launch_bounds__(256) void qk_norm_rotary_append_kernel(
 #pragma unroll
         for (int i = 0; i < 8; ++i) v[i] *= fc * w8[i];
       }
-      if (r0 >= 0 && r0 < 2 * nrot) {
+      if (r0 >= 0 && r0 < 2 * nrot && neighbours) {    // the chunk holds four whole pairs
+        float c8[8];
+        ld_chunk<8>(cs + r0, c8);
+#pragma unroll
+        for (int i = 0; i < 8; i += 2) {
+          const float a = v[i] * c8[i] - v[i + 1] * c8[i + 1];
+          v[i + 1] = v[i + 1] * c8[i] + v[i] * c8[i + 1];
+          v[i] = a;
+        }
+      } else if (r0 >= 0 && r0 < 2 * nrot) {
         const bool first = r0 < nrot;
         const int off = first ? nrot : -nrot, ii = first ? r0 : r0 - nrot;
         float u[8], c8[8], s8[8];
@@ -246,12 +302,14 @@ __global__ __launch_bounds__(256) void qk_norm_rotary_append_kernel(
         v[i] = row[c + i];
         if (ei < nn) v[i] *= fc * wp[ei];
         if (r >= 0 && r < 2 * nrot) {
-          const int ii = r < nrot ? r : r - nrot;
-          const int ej = r < nrot ? ei + nrot : ei - nrot;
+          const bool first = neighbours ? (r & 1) == 0 : r < nrot;
+          const int ii = neighbours ? r >> 1 : (first ? r : r - nrot);
+          const int dist = neighbours ? 1 : nrot;
+          const int ej = first ? ei + dist : ei - dist;
           float u = row[c + i + (ej - ei)];
           if (ej < nn) u *= fc * wp[ej];
           const float cc = cs[2 * ii], sn = cs[2 * ii + 1];
-          v[i] = r < nrot ? v[i] * cc - u * sn : v[i] * cc + u * sn;
+          v[i] = first ? v[i] * cc - u * sn : v[i] * cc + u * sn;
         }
       }
     }
@@ -277,7 +335,8 @@ __global__ __launch_bounds__(256) void attn_keep_window_kernel(
     const int32_t* __restrict__ work_qblk, const float* __restrict__ head_bias,
     const T* __restrict__ gate, int64_t gate_stride, int gate_w, T* __restrict__ out,
     int64_t out_stride,
-    float scale, int window, int keep_first, int sigmoid, int H, int G, int E, int vdim, int BS) {
+    float scale, int window, int keep_first, int sigmoid, int H, int G, int E, int vdim, int BS,
+    float softcap, float out_mult) {
   const int s = work_seq[blockIdx.x];
   if (s < 0) return;
   const int hh = blockIdx.y;
@@ -354,7 +413,7 @@ __global__ __launch_bounds__(256) void attn_keep_window_kernel(
       for (int k = 0; k < 4; ++k) {
         const int jj = tj + 16 * k, j = jb + jj;
         okk[k] = i < nq && jj < nk && j <= pi && (window <= 0 || pi - j < window || j < keep_first);
-        sacc[a][k] = okk[k] ? sacc[a][k] * scale : kNegInfK;
+        sacc[a][k] = okk[k] ? capped(sacc[a][k] * scale, softcap) : kNegInfK;
         mx = fmaxf(mx, sacc[a][k]);
       }
       float alpha = 1.f;
@@ -403,7 +462,7 @@ __global__ __launch_bounds__(256) void attn_keep_window_kernel(
   for (int x = tid; x < nq * vdim; x += 256) {
     const int i = x / vdim, dv = x - i * vdim;
     const int64_t t = q_start[s] + i0 + i;
-    float mul = sigmoid ? 1.f : (ll[i] > 0.f ? 1.0f / ll[i] : 0.f);
+    float mul = sigmoid ? out_mult : (ll[i] > 0.f ? out_mult / ll[i] : 0.f);
     if (gate != nullptr)
       mul /= 1.0f + expf(-ldf(gate + t * gate_stride + (gate_w == 1 ? hh : hh * vdim + dv)));
     stf(out + t * out_stride + (int64_t)hh * vdim + dv, Os[x] * mul);
@@ -426,7 +485,7 @@ __global__ __launch_bounds__(256) void attn_keep_decode_kernel(
     const T* __restrict__ gate, int64_t gate_stride, int gate_w, T* __restrict__ out,
     int64_t out_stride,
     float scale, int window, int keep_first, int sigmoid, int H, int G, int E, int vdim, int BS,
-    int KT) {
+    int KT, float softcap, float out_mult) {
   const int s = blockIdx.x, g = blockIdx.y;
   const int ql = q_len[s];
   const int32_t* bt = block_tables + (int64_t)s * maxb;
@@ -541,7 +600,7 @@ __global__ __launch_bounds__(256) void attn_keep_decode_kernel(
             } else {
               for (int e = 0; e < E; ++e) d0 += qv[e] * kv[e];
             }
-            a = d0 * scale;
+            a = capped(d0 * scale, softcap);
           }
           Ps[row * KT + jj] = a;
           mx = fmaxf(mx, a);
@@ -602,7 +661,7 @@ __global__ __launch_bounds__(256) void attn_keep_decode_kernel(
     __syncthreads();
     for (int hr = wid; hr < R; hr += nw) {
       const int hh = g * R + hr;
-      float mul = sigmoid ? 1.f : (lrow[hr] > 0.f ? 1.0f / lrow[hr] : 0.f);
+      float mul = sigmoid ? out_mult : (lrow[hr] > 0.f ? out_mult / lrow[hr] : 0.f);
       const T* gr = gate == nullptr ? nullptr : gate + (int64_t)t * gate_stride;
       if (gr != nullptr && gate_w == 1) mul /= 1.0f + expf(-ldf(gr + hh));
       for (int dv = lane; dv < vdim; dv += 64) {
@@ -647,7 +706,10 @@ bool launch_qk_norm_rotary_append(bool f32, const void* proj, int64_t stride, co
                                   int k_rot_off, const int32_t* slots, void* k_cache, void* v_cache,
                                   int T, int H, int G, int qw, int kw, int vdim, int v_mode, int BS,
                                   int64_t pool_slots, const float* v_in, float v_take,
-                                  float* v_out, float* q_out, hipStream_t s) {
+                                  float* v_out, float* q_out, bool neighbours, const float* conv_w,
+                                  int taps, float* conv_state, int state_slots,
+                                  const int32_t* row_state, const int32_t* row_back,
+                                  const int32_t* row_fwd, hipStream_t s) {
   const size_t W = (size_t)H * qw + (size_t)G * kw + (v_mode == 0 ? (size_t)G * vdim : 0);
   const size_t lds = (W + 4 + H + G + 4 + 2 * (size_t)nrot + 16) * sizeof(float);
   if (lds > (size_t)kLdsMax) return false;
@@ -665,13 +727,14 @@ bool launch_qk_norm_rotary_append(bool f32, const void* proj, int64_t stride, co
                    stride % 8 == 0 && k_norm_n % 8 == 0 && nrot % 8 == 0 && q_rot_off % 8 == 0 &&
                    k_rot_off % 8 == 0 && al16(proj) && al16(bias) && al16(q_norm_w) &&
                    al16(k_norm_w) && al16(k_cache) && al16(v_cache) && al16(q_out) && al16(v_in) &&
-                   al16(v_out);
+                   al16(v_out) && al16(conv_w) && al16(conv_state);
 #define QKN_GO(TT, CW)                                                                          \
   hipLaunchKernelGGL((qk_norm_rotary_append_kernel<TT, CW>), dim3(T), dim3(256), lds, s,       \
                      (const TT*)proj, stride, bias, q_norm_w, k_norm_w, (int)norm_all, k_norm_n, \
                      eps, pos, inv_freq, nrot, rot_mult, q_rot_off, k_rot_off, slots,           \
                      (TT*)k_cache, (TT*)v_cache, H, G, qw, kw, vdim, v_mode, BS, pool_slots,    \
-                     v_in, 1.0f - v_take, v_take, v_out, q_out)
+                     v_in, 1.0f - v_take, v_take, v_out, q_out, (int)neighbours, conv_w, taps,  \
+                     conv_state, state_slots, row_state, row_back, row_fwd)
   if (f32) {
     if (vec) QKN_GO(float, 8);
     else QKN_GO(float, 1);
@@ -689,7 +752,7 @@ bool launch_attn_keep_window(bool f32, const float* q, const void* k_cache, cons
                              const int32_t* work_qblk, int W, const float* head_bias,
                              const void* gate, int64_t gate_stride, int gate_w, void* out,
                              int64_t out_stride, float scale, int window, int keep_first, bool sigmoid, int H, int G,
-                             int E, int vdim, int BS, hipStream_t s) {
+                             int E, int vdim, int BS, float softcap, float out_mult, hipStream_t s) {
   const size_t lds = ((size_t)KQB * (KEC + 1) + (size_t)KKT * (KEC + 1) + (size_t)KQB * (KKT + 1) +
                       (size_t)KQB * vdim + 2 * KQB) * sizeof(float);
   if (lds > (size_t)kLdsMax) return false;
@@ -705,13 +768,13 @@ bool launch_attn_keep_window(bool f32, const float* q, const void* k_cache, cons
                        (const float*)k_cache, (const float*)v_cache, vrs, bt, maxb, q_start, q_len,
                        kv_len, work_seq, work_qblk, head_bias, (const float*)gate, gate_stride, gate_w,
                        (float*)out, out_stride, scale, window, keep_first, (int)sigmoid, H, G, E,
-                       vdim, BS);
+                       vdim, BS, softcap, out_mult);
   else
     hipLaunchKernelGGL(attn_keep_window_kernel<bf16_t>, dim3(W, H), dim3(256), lds, s, q,
                        (const bf16_t*)k_cache, (const bf16_t*)v_cache, vrs, bt, maxb, q_start, q_len,
                        kv_len, work_seq, work_qblk, head_bias, (const bf16_t*)gate, gate_stride, gate_w,
                        (bf16_t*)out, out_stride, scale, window, keep_first, (int)sigmoid, H, G, E,
-                       vdim, BS);
+                       vdim, BS, softcap, out_mult);
   return true;
 }
 
@@ -727,7 +790,8 @@ int launch_attn_keep_decode(bool f32, const float* q, const void* k_cache, const
                             const int32_t* q_len, const int32_t* kv_len, int NA, int max_rows,
                             const float* head_bias, const void* gate, int64_t gate_stride,
                             int gate_w, void* out, int64_t out_stride, float scale, int window, int keep_first,
-                            bool sigmoid, int H, int G, int E, int vdim, int BS, hipStream_t s) {
+                            bool sigmoid, int H, int G, int E, int vdim, int BS, float softcap,
+                            float out_mult, hipStream_t s) {
   const int R = H / G;
   int KT = 64;
   while (KT >= 16 && attn_keep_decode_floats(R, E, vdim, KT) * 4 > 80 * 1024) KT >>= 1;
@@ -749,12 +813,14 @@ int launch_attn_keep_decode(bool f32, const float* q, const void* k_cache, const
     hipLaunchKernelGGL(attn_keep_decode_kernel<float>, grid, dim3(256), lds, s, q,
                        (const float*)k_cache, (const float*)v_cache, vrs, bt, maxb, q_start, q_len,
                        kv_len, head_bias, (const float*)gate, gate_stride, gate_w, (float*)out, out_stride,
-                       scale, window, keep_first, (int)sigmoid, H, G, E, vdim, BS, KT);
+                       scale, window, keep_first, (int)sigmoid, H, G, E, vdim, BS, KT, softcap,
+                       out_mult);
   else
     hipLaunchKernelGGL(attn_keep_decode_kernel<bf16_t>, grid, dim3(256), lds, s, q,
                        (const bf16_t*)k_cache, (const bf16_t*)v_cache, vrs, bt, maxb, q_start, q_len,
                        kv_len, head_bias, (const bf16_t*)gate, gate_stride, gate_w, (bf16_t*)out, out_stride,
-                       scale, window, keep_first, (int)sigmoid, H, G, E, vdim, BS, KT);
+                       scale, window, keep_first, (int)sigmoid, H, G, E, vdim, BS, KT, softcap,
+                       out_mult);
   return KT;
 }
 

@@ -59,7 +59,8 @@ __global__ __launch_bounds__(128 * HPW) void attn_keep_mfma_kernel(
     const int32_t* __restrict__ kv_len, const int32_t* __restrict__ work_seq,
     const int32_t* __restrict__ work_qblk, const float* __restrict__ head_bias,
     const bf16_t* __restrict__ gate, int64_t gate_stride, int gate_w,
-    bf16_t* __restrict__ out, int64_t out_stride, float scale, int window, int keep_first, int sigmoid, int H, int G) {
+    bf16_t* __restrict__ out, int64_t out_stride, float scale, int window, int keep_first, int sigmoid, int H, int G,
+    float softcap, float out_mult) {
   constexpr int E = 32 * DK, vdim = 16 * DV, NT = 128 * HPW;
   constexpr int KRS = E + 8;                       // shorts per key row in LDS (+ 16 bytes)
   constexpr int VRS = SHARED ? KRS : vdim + 8;     // shorts per value row
@@ -192,6 +193,17 @@ __global__ __launch_bounds__(128 * HPW) void attn_keep_mfma_kernel(
           sc[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(kfr), as_bf16x8(qlo[ks]), sc[kt], 0, 0, 0);
       }
     }
+    // the scaled scores, capped where a cap is given: c tanh(s / c) = c - 2 c / (exp(2 s / c) + 1)
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt) sc[kt] *= scale;
+    if (softcap > 0.f) {
+      const float two_c = 2.f * softcap, inv = 2.f / softcap;
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          sc[kt][i] = softcap - two_c * __builtin_amdgcn_rcpf(__expf(sc[kt][i] * inv) + 1.f);
+    }
     float pv[8];
     float alpha = 1.f;
     if (sigmoid) {
@@ -201,7 +213,7 @@ __global__ __launch_bounds__(128 * HPW) void attn_keep_mfma_kernel(
         for (int i = 0; i < 4; ++i) {
           const int j = jb + kt * 16 + grp * 4 + i;
           const bool ok = qlive && j <= pi && (window <= 0 || pi - j < window || j < keep_first);
-          pv[kt * 4 + i] = ok ? 1.0f / (1.0f + __expf(-(sc[kt][i] * scale + hb))) : 0.f;
+          pv[kt * 4 + i] = ok ? 1.0f / (1.0f + __expf(-(sc[kt][i] + hb))) : 0.f;
         }
     } else {
       float mx = kNegInfW;
@@ -211,7 +223,7 @@ __global__ __launch_bounds__(128 * HPW) void attn_keep_mfma_kernel(
         for (int i = 0; i < 4; ++i) {
           const int j = jb + kt * 16 + grp * 4 + i;
           const bool ok = qlive && j <= pi && (window <= 0 || pi - j < window || j < keep_first);
-          sc[kt][i] = ok ? sc[kt][i] * scale : kNegInfW;
+          sc[kt][i] = ok ? sc[kt][i] : kNegInfW;
           mx = fmaxf(mx, sc[kt][i]);
         }
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
@@ -256,7 +268,7 @@ __global__ __launch_bounds__(128 * HPW) void attn_keep_mfma_kernel(
   }
   // lane (col, grp) holds value channels 16 m + 4 grp .. + 3 of its column: 8-byte stores
   if (qlive) {
-    float mul = sigmoid ? 1.f : (lrun > 0.f ? 1.0f / lrun : 0.f);
+    float mul = sigmoid ? out_mult : (lrun > 0.f ? out_mult / lrun : 0.f);
     if (gate != nullptr && gate_w == 1) mul /= 1.0f + __expf(-ldf(gate + t * gate_stride + hh));
     // a gate column per output: four neighbouring logits per 16-channel block, 8-byte reads
     const bf16_t* grow = gate != nullptr && gate_w > 1
@@ -314,6 +326,7 @@ struct KeepArgs {
   bool sigmoid;
   int H, G;
   int NA, short_rows;      // decode rows: sequences, and the most rows any of them has (0: work items)
+  float softcap, out_mult;
   hipStream_t s;
 };
 
@@ -338,7 +351,7 @@ static void launch_keep_mfma_one(const KeepArgs& a) {
                      (const bf16_t*)a.v_cache, a.vrs, a.bt, a.maxb, a.q_start, a.q_len, a.kv_len,
                      a.work_seq, a.work_qblk, a.head_bias, (const bf16_t*)a.gate, a.gate_stride,
                      a.gate_w, (bf16_t*)a.out, a.out_stride, a.scale, a.window, a.keep_first, (int)a.sigmoid,
-                     a.H, a.G);
+                     a.H, a.G, a.softcap, a.out_mult);
 }
 
 template <int DK, int DV, bool SHARED>
@@ -355,12 +368,12 @@ bool launch_attn_keep_mfma(const float* q, const void* k_cache, const void* v_ca
                            const void* gate, int64_t gate_stride, int gate_w, void* out,
                            int64_t out_stride, float scale, int window, int keep_first, bool sigmoid, int H, int G,
                            int E, int vdim, int BS, bool shared, int NA, int short_rows,
-                           hipStream_t s) {
+                           float softcap, float out_mult, hipStream_t s) {
   if (!keep_mfma_ok(E, vdim, BS, shared)) return false;
   if (short_rows > 0 ? NA == 0 : W == 0) return true;
   const KeepArgs a{q, k_cache, v_cache, vrs, bt, maxb, q_start, q_len, kv_len, work_seq, work_qblk,
                    W, head_bias, gate, gate_stride, gate_w, out, out_stride, scale, window, keep_first,
-                   sigmoid, H, G, NA, short_rows, s};
+                   sigmoid, H, G, NA, short_rows, softcap, out_mult, s};
   const int DK = E / 32, DV = vdim / 16;
   if (shared) {
     if (DK == 3) launch_keep_mfma_heads<3, 4, true>(a);

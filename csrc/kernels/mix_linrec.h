@@ -25,7 +25,8 @@ struct LinrecArgs {
   float* state;                     // [2 slots, H, dim, vdim]
   const int32_t *row_state, *row_back, *row_fwd, *pos, *run_rows;
   int runs;
-  void* out;                        // [T, H vdim]
+  void* out;                        // [T, H vdim], row stride os
+  int64_t os;
   int T, H, rep, dim, vdim, slots;
 };
 

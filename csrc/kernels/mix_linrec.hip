@@ -41,7 +41,7 @@ __global__ __launch_bounds__(256) void gated_linrec_kernel(
     const int32_t* __restrict__ row_state,
     const int32_t* __restrict__ row_back, const int32_t* __restrict__ row_fwd,
     const int32_t* __restrict__ pos, const int32_t* __restrict__ run_rows, TG* __restrict__ out,
-    int H, int rep, int dim, int vdim, int slots) {
+    int64_t o_stride, int H, int rep, int dim, int vdim, int slots) {
   const int t0 = run_rows != nullptr ? run_rows[blockIdx.x] : (int)blockIdx.x;
   const int h = blockIdx.y;
   if (t0 < 0 || row_back[t0] != 0) return;
@@ -173,7 +173,7 @@ __global__ __launch_bounds__(256) void gated_linrec_kernel(
     const float ss = block_sum(vlive ? o * o : 0.f, scratch);
     if (vlive) {
       const float act = gate_sigmoid ? 1.0f / (1.0f + expf(-gj)) : gj / (1.0f + expf(-gj));
-      stf(out + (int64_t)(t0 + a) * H * vdim + vc, o / sqrtf(ss / (float)vdim + eps) * my_nw * act);
+      stf(out + (int64_t)(t0 + a) * o_stride + vc, o / sqrtf(ss / (float)vdim + eps) * my_nw * act);
     }
   }
   if (code >= 0 && vlive) {
@@ -211,8 +211,8 @@ void launch_decay_from_logits(float* z, int64_t z_stride, const float* rate, con
 template <typename TG>
 __global__ __launch_bounds__(256) void linrec_finish_kernel(
     const float* __restrict__ raw, const TG* __restrict__ gate, int64_t g_stride,
-    int gate_sigmoid, const float* __restrict__ norm_w, float eps, TG* __restrict__ out, int T,
-    int H, int vdim) {
+    int gate_sigmoid, const float* __restrict__ norm_w, float eps, TG* __restrict__ out,
+    int64_t o_stride, int T, int H, int vdim) {
   const int lane = threadIdx.x & 63;
   const int64_t item = (int64_t)blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
   if (item >= (int64_t)T * H) return;
@@ -226,7 +226,7 @@ __global__ __launch_bounds__(256) void linrec_finish_kernel(
   for (int c = lane; c < vdim; c += 64) {
     const float gj = ldf(gate + t * g_stride + (int64_t)h * vdim + c);
     const float act = gate_sigmoid ? 1.0f / (1.0f + expf(-gj)) : gj / (1.0f + expf(-gj));
-    stf(out + item * vdim + c, r[c] * inv * norm_w[c] * act);
+    stf(out + t * o_stride + (int64_t)h * vdim + c, r[c] * inv * norm_w[c] * act);
   }
 }
 
@@ -352,7 +352,7 @@ static void launch_linrec_one(const LinrecArgs& a, hipStream_t s) {
                      a.rate, a.zbias, a.zsign, (const TG*)a.beta, a.bs, (const TG*)a.gate, a.gs,
                      a.gate_sigmoid, a.norm_w, a.eps, a.q_scale, a.decay_ready, a.raw, a.state,
                      a.row_state, a.row_back,
-                     a.row_fwd, a.pos, a.run_rows, (TG*)a.out, a.H, a.rep, a.dim, a.vdim, a.slots);
+                     a.row_fwd, a.pos, a.run_rows, (TG*)a.out, a.os, a.H, a.rep, a.dim, a.vdim, a.slots);
 }
 
 template <typename TI, typename TG, bool DELTA>
@@ -390,11 +390,11 @@ void launch_gated_linrec(bool in_f32, bool act_f32, bool delta, const LinrecArgs
     if (act_f32)
       hipLaunchKernelGGL(linrec_finish_kernel<float>, grid, dim3(256), 0, s, a.raw,
                          (const float*)a.gate, a.gs, a.gate_sigmoid, a.norm_w, a.eps,
-                         (float*)a.out, a.T, a.H, a.vdim);
+                         (float*)a.out, a.os, a.T, a.H, a.vdim);
     else
       hipLaunchKernelGGL(linrec_finish_kernel<bf16_t>, grid, dim3(256), 0, s, a.raw,
                          (const bf16_t*)a.gate, a.gs, a.gate_sigmoid, a.norm_w, a.eps,
-                         (bf16_t*)a.out, a.T, a.H, a.vdim);
+                         (bf16_t*)a.out, a.os, a.T, a.H, a.vdim);
   }
 }
 

@@ -64,7 +64,8 @@ class LayeredKVCache:
       window_attention   K and V pools like ``attention``;
       rope_latent_attention   like ``latent_attention`` with rows ``[latent | rotated key
                          part]``, ``kv_rank + rot_dim`` wide;
-      wkv, gla, channel_delta, mlstm   no pages.
+      wkv, gla, channel_delta, mlstm   no pages;
+      parallel           the pages of its one part that has any.
     Per-sequence state lives in slots; a sequence owns one while it runs (native core).  Every
     state pool is double buffered: a step reads half ``gen & 1`` of the slot and writes the
     other, so rows of one launch never read what the launch writes.  ``state``: the input
@@ -72,8 +73,9 @@ class LayeredKVCache:
     ``layer_state[i]``: name -> ``[2 * slots, ...]`` fp32 for what ``cfg.state_shapes(i)``
     lists (a wkv layer's matrices and its previous input row; a gla or channel_delta
     layer's matrices, and the convolutions' last inputs; an mlstm layer's matrices, key sums
-    and running maxima; with ``cfg.token_shift`` every
-    layer's previous normed input row)."""
+    and running maxima; the convolutions' last inputs of a window_attention layer that has one;
+    for a parallel layer what its parts hold, the names preceded by the part's index; with
+    ``cfg.token_shift`` every layer's previous normed input row)."""
 
     def __init__(self, cfg, num_blocks: int, device, num_slots: int, block_size: int = 32,
                  dtype=torch.bfloat16, prefix_cache: bool = False):
@@ -85,7 +87,7 @@ class LayeredKVCache:
         self.k, self.v = [], []
         runs = tuple(getattr(cfg, "runs", range(cfg.n_layers)))
         for li in runs:
-            m = cfg.layers[li].mixer
+            m = cfg.layers[li].mixer.paged
             if m.kind == "attention":
                 self.k.append(mk((num_blocks, m.kv_heads, block_size, m.dim), dtype=dtype, device=device))
                 self.v.append(mk((num_blocks, m.kv_heads, block_size, m.vdim), dtype=dtype, device=device))

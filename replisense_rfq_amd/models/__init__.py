@@ -24,4 +24,8 @@ def layered_model_class(architecture: str):
         from .modepel import ModepelLM
 
         return ModepelLM
+    if architecture == "Minerax":
+        from .minerax import MineraxLM
+
+        return MineraxLM
     raise KeyError(f"no model class for architecture {architecture!r}")

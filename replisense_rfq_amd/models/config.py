@@ -109,7 +109,8 @@ class MixerSpec:
     ``rope_latent_attention``: latent attention whose heads also hold ``rot_dim`` rotated
     query dimensions that meet ONE rotated key part shared by all heads; a token caches
     its latent and that key part (``kv_rank + rot_dim`` numbers); softmax with a sink and a
-    sigmoid output gate per head; ``kv_from`` as for ``latent_attention``.
+    sigmoid output gate per head, or with ``out_gate`` per output; ``window`` and ``kv_from`` as
+    for the other kinds.
     ``window_attention``: grouped heads with ``qk_norm`` over each head (``head``) or over the
     whole projection (``all``), half-split rotation of the first ``rot_dims`` dimensions,
     position i sees j <= i with i - j < ``window`` or j < ``keep_first`` (window 0: plain
@@ -117,9 +118,13 @@ class MixerSpec:
     ``bias``: the projections have biases; ``v_is_k``: the values are the keys as projected;
     ``sink`` = ``unit``: the softmax's denominator holds an added 1; ``v_mix``: the values are
     blended with those of the first layer that has it (which stay as projected); ``out_gate``: a
-    sigmoid gate per output.
+    sigmoid gate per output; ``conv``: q, k and v pass a causal convolution of that many taps
+    before norm and rotation; ``softcap`` > 0: scores <- softcap tanh(score / softcap).
     ``mlstm``: ``heads`` recurrent heads with a ``dim`` x ``vdim`` matrix memory, a ``dim``-wide
     key sum and a running maximum, exponential gates whose logits are capped at ``gate_cap``.
+    ``parallel``: the mixers in ``parts`` side by side on the same input, their results summed
+    with the factors ``part_scales``; at most one of them has cache pages.
+    ``rot_neighbours``: dimension 2i turns with 2i + 1 instead of i with i + rot_dims / 2.
     The rotating kinds take their frequencies from ``rot_base`` and ``rot_scaling``: () for
     none, ("yarn", factor, original, fast, slow) or ("banded", factor, original, low,
     high)."""
@@ -150,10 +155,24 @@ class MixerSpec:
     v_mix: bool = False
     out_gate: bool = False
     gate_cap: float = 0.0
+    softcap: float = 0.0
+    rot_neighbours: bool = False
+    parts: tuple = ()
+    part_scales: tuple = ()
 
     @property
     def group(self) -> int:
         return self.heads // self.kv_heads
+
+    @property
+    def mixers(self) -> tuple:
+        """The mixers that do the work: the parts of a parallel mixer, else the mixer itself."""
+        return self.parts if self.kind == "parallel" else (self,)
+
+    @property
+    def paged(self) -> "MixerSpec":
+        """The part that owns cache pages (the mixer itself where it has no parts)."""
+        return next((p for p in self.mixers if p.kind.endswith("attention")), self.mixers[0])
 
 
 @dataclass(frozen=True)
@@ -168,7 +187,8 @@ class MlpSpec:
     normed powers, down projection.  ``router`` = ``grouped_softmax``: softmax over the experts and
     ``identity`` further router outputs whose "expert" is the input itself, a correction in the
     choice, groups ranked by their largest choice score, weights times ``router_scale``; the shared
-    expert is then gated by one logit per token."""
+    expert is then gated by one logit per token.  ``gelu_glu``: down projection of the tanh form of
+    gelu of the gate times the up projection."""
     kind: str = "dense"
     ff: int = 256
     limit: float = 7.0
@@ -213,6 +233,10 @@ class LayeredConfig:
     # every layer's mixer reads h + (h' - h) * shift, h' the previous token's normed input
     # (one row of per-sequence state per layer)
     token_shift: bool = False
+    # > 1 residual streams: a sublayer reads a weighted sum of them, its result joins each with a
+    # weight of its own, and a matrix mixes them at the same time
+    streams: int = 1
+    logit_scale: float = 1.0
 
     @property
     def n_layers(self) -> int:
@@ -245,33 +269,34 @@ class LayeredConfig:
     def params(self) -> int:
         d, n = self.hidden, 0
         for ly in self.layers:
-            m = ly.mixer
-            if m.kind == "attention":
-                n += d * (m.heads * m.dim + m.kv_heads * (m.dim + m.vdim)) + m.heads * m.vdim * d
-                n += 2 * m.dim + m.heads * m.heads + m.heads + 6 * d + 2 * d * self.canon_taps
-            elif m.kind == "latent_attention":
-                n += d * m.q_rank + m.q_rank * m.heads * m.dim + m.heads * m.vdim * d
-                n += m.kv_rank * m.heads * (m.dim + m.vdim) + (d * m.kv_rank if m.kv_from < 0 else 0)
-            elif m.kind == "diff_attention":
-                n += d * (2 * m.dim * (m.heads + m.kv_heads) + m.kv_heads * m.vdim + m.heads)
-                n += m.heads * m.vdim * d
-            elif m.kind == "rope_latent_attention":
-                n += d * m.heads * (m.dim + m.rot_dim + 1) + m.heads * m.vdim * d
-                n += m.kv_rank * m.heads * (m.dim + m.vdim)
-                n += d * (m.kv_rank + m.rot_dim) if m.kv_from < 0 else 0
-            elif m.kind == "window_attention":
-                n += d * (m.heads * m.dim + m.kv_heads * (m.dim + (0 if m.v_is_k else m.vdim)))
-                n += m.heads * m.vdim * d * (2 if m.out_gate else 1)
-            elif m.kind == "mlstm":
-                n += d * m.heads * (2 * m.dim + 3 * m.vdim + 2)
-            elif m.kind == "gla":
-                n += 2 * d * m.heads * (m.dim + m.vdim) + m.heads * m.vdim * d
-                n += self.decay_rank * (d + m.heads * m.dim)
-            elif m.kind == "channel_delta":
-                n += d * (2 * m.kv_heads * m.dim + m.heads * m.vdim + m.heads) + m.heads * m.vdim * d
-                n += self.decay_rank * (d + m.heads * m.dim) + self.gate_rank * (d + m.heads * m.vdim)
-            else:
-                n += 5 * d * m.heads * m.dim + 2 * d * self.decay_rank
+            for m in ly.mixer.mixers:
+                if m.kind == "attention":
+                    n += d * (m.heads * m.dim + m.kv_heads * (m.dim + m.vdim)) + m.heads * m.vdim * d
+                    n += 2 * m.dim + m.heads * m.heads + m.heads + 6 * d + 2 * d * self.canon_taps
+                elif m.kind == "latent_attention":
+                    n += d * m.q_rank + m.q_rank * m.heads * m.dim + m.heads * m.vdim * d
+                    n += m.kv_rank * m.heads * (m.dim + m.vdim) + (d * m.kv_rank if m.kv_from < 0 else 0)
+                elif m.kind == "diff_attention":
+                    n += d * (2 * m.dim * (m.heads + m.kv_heads) + m.kv_heads * m.vdim + m.heads)
+                    n += m.heads * m.vdim * d
+                elif m.kind == "rope_latent_attention":
+                    n += d * m.heads * (m.dim + m.rot_dim + (m.vdim if m.out_gate else 1))
+                    n += m.heads * m.vdim * d
+                    n += m.kv_rank * m.heads * (m.dim + m.vdim)
+                    n += d * (m.kv_rank + m.rot_dim) if m.kv_from < 0 else 0
+                elif m.kind == "window_attention":
+                    n += d * (m.heads * m.dim + m.kv_heads * (m.dim + (0 if m.v_is_k else m.vdim)))
+                    n += m.heads * m.vdim * d * (2 if m.out_gate else 1)
+                elif m.kind == "mlstm":
+                    n += d * m.heads * (2 * m.dim + 3 * m.vdim + 2)
+                elif m.kind == "gla":
+                    n += 2 * d * m.heads * (m.dim + m.vdim) + m.heads * m.vdim * d
+                    n += self.decay_rank * (d + m.heads * m.dim)
+                elif m.kind == "channel_delta":
+                    n += d * (2 * m.kv_heads * m.dim + m.heads * m.vdim + m.heads) + m.heads * m.vdim * d
+                    n += self.decay_rank * (d + m.heads * m.dim) + self.gate_rank * (d + m.heads * m.vdim)
+                else:
+                    n += 5 * d * m.heads * m.dim + 2 * d * self.decay_rank
             f = ly.mlp
             if f is not None and f.kind == "moe":
                 n += 3 * d * (f.ff * f.experts + f.shared_ff) + d * (f.experts + f.identity)
@@ -282,7 +307,7 @@ class LayeredConfig:
     def kv_bytes_per_token(self, tp: int = 1, dtype_bytes: int = 2) -> int:
         n = 0
         for li in self.runs:
-            m = self.layers[li].mixer
+            m = self.layers[li].mixer.paged
             if m.kind == "attention":
                 n += m.kv_heads * (m.dim + m.vdim)
             elif m.kind == "diff_attention":
@@ -297,10 +322,17 @@ class LayeredConfig:
 
     def state_shapes(self, li: int) -> dict:
         """Per-sequence recurrent state of layer ``li`` besides cache pages and the input
-        convolutions: name -> shape of one slot (fp32)."""
+        convolutions: name -> shape of one slot (fp32); the names of a parallel mixer's parts
+        start with the part's index."""
         m = self.layers[li].mixer
         if self.token_shift:
             return {"prev": (self.hidden,)}
+        if m.kind == "parallel":
+            return {f"{i}.{name}": shape for i, p in enumerate(m.parts)
+                    for name, shape in self._mixer_state(p).items()}
+        return self._mixer_state(m)
+
+    def _mixer_state(self, m: MixerSpec) -> dict:
         if m.kind == "wkv":
             return {"wkv": (m.heads, m.dim, m.dim), "prev": (self.hidden,)}
         if m.kind == "mlstm":
@@ -310,6 +342,8 @@ class LayeredConfig:
         if m.kind == "channel_delta":
             return {"S": (m.heads, m.dim, m.vdim),
                     "conv": (max(0, m.conv - 1), 2 * m.kv_heads * m.dim + m.heads * m.vdim)}
+        if m.kind == "window_attention" and m.conv > 0:
+            return {"conv": (m.conv - 1, m.heads * m.dim + m.kv_heads * (m.dim + m.vdim))}
         return {}
 
     def to_dict(self):
@@ -561,6 +595,89 @@ def modepel_from_json(d: dict, name: str | None = None) -> LayeredConfig:
                          max_position=int(d.get("max_position", 8192)))
 
 
+def _rot(m: dict, i: int, width: int) -> dict:
+    """MixerSpec fields of a mixer's ``rot`` entry; the rotated dimensions fit into ``width``."""
+    rot = m.get("rot") or {}
+    dims = int(rot.get("dims", 0))
+    if dims % 2 or not 0 <= dims <= width:
+        raise ValueError(f"layer {i}: rot.dims must be even and at most {width}")
+    return dict(rot_dims=dims, rot_base=float(rot.get("base", 10000.0)),
+                rot_scaling=_rot_scaling(rot.get("scaling")))
+
+
+def minerax_from_json(d: dict, name: str | None = None) -> LayeredConfig:
+    """config.json of a Minerax checkpoint: vocab, width, norm.eps, streams, logit_scale and
+    ``layers``: type ``parallel`` (left: heads, kv_heads, dim, vdim, conv, scale, softcap, rot;
+    right: heads, kv_heads, dim, vdim, conv; left_scale, right_scale) or ``latent_attention``
+    (heads, dim, rot_dim, vdim, kv_rank, scale, rot, mask.size), each with an ``mlp`` of kind
+    ``dense`` (ff) or null."""
+    layers = []
+    for i, ly in enumerate(d["layers"]):
+        m, kind = ly["mixer"], ly["type"]
+        if kind == "parallel":
+            a, b = m["left"], m["right"]
+            left = MixerSpec("window_attention", int(a["heads"]), int(a["kv_heads"]), int(a["dim"]),
+                             int(a["vdim"]), float(a["scale"]), conv=int(a["conv"]), qk_norm="all",
+                             softcap=float(a.get("softcap") or 0.0), **_rot(a, i, int(a["dim"])))
+            right = MixerSpec("channel_delta", int(b["heads"]), int(b["kv_heads"]), int(b["dim"]),
+                              int(b["vdim"]), float(b["dim"]) ** -0.5, conv=int(b["conv"]))
+            if left.conv < 1 or right.conv < 1:
+                raise ValueError(f"layer {i}: a convolution needs at least one tap")
+            mixer = MixerSpec("parallel", parts=(left, right),
+                              part_scales=(float(m["left_scale"]), float(m["right_scale"])))
+        elif kind == "latent_attention":
+            mixer = MixerSpec("rope_latent_attention", int(m["heads"]), 1, int(m["dim"]), int(m["vdim"]),
+                              float(m["scale"]), kv_rank=int(m["kv_rank"]), rot_dim=int(m["rot_dim"]),
+                              window=int((m.get("mask") or {}).get("size", 0)), rot_neighbours=True,
+                              out_gate=True, **_rot(m, i, int(m["rot_dim"])))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+        for p in mixer.mixers:
+            if p.heads % p.kv_heads:
+                raise ValueError(f"layer {i}: heads must be a multiple of kv_heads")
+        f = ly.get("mlp")
+        if f is not None and f.get("kind") != "dense":
+            raise ValueError(f"layer {i}: unknown feed-forward kind {f.get('kind')!r}")
+        layers.append(LayerSpec(mixer, None if f is None else MlpSpec("gelu_glu", int(f["ff"]), 0.0)))
+    streams = int(d.get("streams", 1))
+    if streams < 1:
+        raise ValueError("streams must be at least 1")
+    return LayeredConfig(name=name or d["architecture"].lower(), architecture=d["architecture"],
+                         vocab_size=int(d["vocab"]), hidden=int(d["width"]), layers=tuple(layers),
+                         rms_eps=float(d["norm"]["eps"]), canon_taps=0,
+                         max_position=int(d.get("max_position", 8192)), streams=streams,
+                         logit_scale=float(d.get("logit_scale", 1.0)))
+
+
+def minerax_layers(order, heads, kv_heads, dim, vdim, ff, conv=3, softcap=30.0, rec_heads=None,
+                   rec_kv_heads=None, rec_dim=None, rec_vdim=None, rec_conv=4, scales=(0.6, 0.9),
+                   latent_heads=None, latent_dim=None, latent_vdim=None, kv_rank=0, rot_dim=0, window=0,
+                   rot_dims=None, rot_base=10000.0, yarn=(), scale=None):
+    """Layers of the kinds named in ``order``: "p" attention and delta rule side by side, "l"
+    windowed latent attention with a rotated key part."""
+    out = []
+    rh = rec_heads or heads
+    rd = rec_dim or dim
+    lh, ld = latent_heads or heads, latent_dim or dim
+    scaling = ("yarn",) + tuple(yarn) if yarn else ()
+    for c in order:
+        if c == "p":
+            left = MixerSpec("window_attention", heads, kv_heads, dim, vdim, scale or dim ** -0.5,
+                             conv=conv, qk_norm="all", softcap=softcap,
+                             rot_dims=dim if rot_dims is None else rot_dims, rot_base=rot_base,
+                             rot_scaling=scaling)
+            right = MixerSpec("channel_delta", rh, rec_kv_heads or rh, rd, rec_vdim or vdim, rd ** -0.5,
+                              conv=rec_conv)
+            m = MixerSpec("parallel", parts=(left, right), part_scales=tuple(scales))
+        else:
+            m = MixerSpec("rope_latent_attention", lh, 1, ld, latent_vdim or vdim,
+                          scale or (ld + rot_dim) ** -0.5, kv_rank=kv_rank, rot_dim=rot_dim,
+                          rot_dims=rot_dim, rot_base=rot_base, rot_scaling=scaling, window=window,
+                          rot_neighbours=True, out_gate=True)
+        out.append(LayerSpec(m, MlpSpec("gelu_glu", ff, 0.0) if ff else None))
+    return tuple(out)
+
+
 def modepel_layers(order, heads, kv_heads, dim, vdim, ff, experts=0, top=0, expert_ff=0, identity=0,
                    groups=0, keep=0, shared_ff=0, router_scale=1.0, rot_dims=None, rot_base=10000.0,
                    scale=None, gate_cap=15.0, rec_heads=None, rec_dim=None, rec_vdim=None, moe_from=1):
@@ -693,13 +810,22 @@ TINY_MODEPEL = LayeredConfig("tiny-modepel", architecture="Modepel", vocab_size=
                                                    shared_ff=56, router_scale=1.3, rot_dims=8,
                                                    rot_base=5000.0, gate_cap=9.0, rec_heads=3,
                                                    rec_dim=20, rec_vdim=28))
+# both kinds of layers; sizes that differ wherever the design allows
+TINY_MINERAX = LayeredConfig("tiny-minerax", architecture="Minerax", vocab_size=336, hidden=96,
+                             canon_taps=0, decay_rank=8, gate_rank=12, streams=3, logit_scale=1.5,
+                             layers=minerax_layers("plp", 6, 2, 16, 24, 160, conv=4, softcap=12.0,
+                                                   rec_heads=4, rec_kv_heads=2, rec_dim=20, rec_vdim=28,
+                                                   rec_conv=3, scales=(0.7, 1.2), latent_heads=5,
+                                                   latent_dim=12, kv_rank=40, rot_dim=8, window=21,
+                                                   rot_dims=8, rot_base=5000.0,
+                                                   yarn=(3.0, 64.0, 16.0, 2.0)))
 CONFIGS.update({c.name: c for c in (TINY_LIVISUN, LIVISUN_8B, TINY_NUMALORN, TINY_BILOLIX,
-                                    TINY_NUTITAR, TINY_MODEPEL)})
+                                    TINY_NUTITAR, TINY_MODEPEL, TINY_MINERAX)})
 
 # config.json "architecture" -> reader
 ARCHITECTURES = {"Livisun": LayeredConfig.from_json, "Numalorn": numalorn_from_json,
                  "Bilolix": bilolix_from_json, "Nutitar": nutitar_from_json,
-                 "Modepel": modepel_from_json}
+                 "Modepel": modepel_from_json, "Minerax": minerax_from_json}
 
 
 def load_config(path: str):

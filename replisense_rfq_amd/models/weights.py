@@ -301,6 +301,8 @@ def load_layered_safetensors(path: str, cfg, device, dtype=torch.bfloat16) -> di
         return _nutitar_assemble(ck.full, lambda k: k in ck, cfg, device, dtype)
     if cfg.architecture == "Modepel":
         return _modepel_assemble(ck.full, lambda k: k in ck, cfg, device, dtype)
+    if cfg.architecture == "Minerax":
+        return _minerax_assemble(ck.full, lambda k: k in ck, cfg, device, dtype)
     w = {"embed": ck.full("embed").to(dtype).to(device), "lm_head": ck.full("head").to(dtype).to(device),
          "final_norm": ck.full("final.norm").float().to(device), "vocab_start": 0, "layers": []}
     for i, ly in enumerate(cfg.layers):
@@ -1014,5 +1016,172 @@ def init_modepel_weights(cfg, device, dtype=torch.bfloat16, seed: int = 0,
 
 def modepel_from_full(full: dict, cfg, device, dtype=torch.bfloat16) -> dict:
     w = _modepel_assemble(lambda k: full[k], lambda k: k in full, cfg, device, dtype)
+    w["full"] = full
+    return w
+
+
+# --------------------------------------------------------------------------
+# Minerax.  Checkpoint names:
+#   embed, head [V, d]; final.norm, l<i>.norm1 | norm2 [d]; l<i>.hc1 | hc2 .in | .out [S]  .mix [S, S]
+#     (S streams; norm2 and hc2 only in layers with a feed-forward)
+#   parallel: l<i>.mix.left.q [H*dim, d]  .k [G*dim, d]  .v [G*vdim, d]  .q.norm [H*dim]  .k.norm
+#     [G*dim]  .{q,k,v}.conv [rows, taps]  .o [d, H*vdim];  l<i>.mix.right.q | k | v (+ .conv)  .b [H, d]
+#     .A_log [H]  .a1 [rank, d]  .a2 [H*dim, rank]  .dt_bias [H*dim]  .g1 [rank, d]  .g2 [H*vdim, rank]
+#     .norm [vdim]  .o [d, H*vdim]
+#   latent_attention: l<i>.mix.q [H*(dim+rot_dim), d]  .dkv [kv_rank+rot_dim, d]  .dkv.norm [kv_rank]
+#     .uk [H*dim, kv_rank]  .uv [H*vdim, kv_rank]  .sink [H]  .g [H*vdim, d]  .o [d, H*vdim]
+#   feed-forward: l<i>.mlp.gate | up [F, d]  .down [d, F]
+# Loaded layout per layer: one fused input projection "proj" with the first column of every part of
+# it in "seg"; a parallel layer's two output projections side by side in "o" (their inputs lie
+# side by side as well, each already times its mixer's factor: the right one's is part of its norm
+# weight "gn"); the attention's taps as rows "conv_l" [taps, channels], the delta rule's per channel
+# "conv_r" [channels, taps]; uk [H, dim, R] and uv^T [H, R, vdim]; the logits' factor is part of
+# the final norm's weight.
+def _minerax_assemble(get, has, cfg, device, dtype) -> dict:
+    d, S = cfg.hidden, cfg.streams
+
+    def mat(name, rows, cols):
+        t = get(name)
+        if tuple(t.shape) != (rows, cols):
+            raise ValueError(f"tensor {name}: shape {tuple(t.shape)}, expected {(rows, cols)}")
+        return t.to(dtype)
+
+    def lowrank(name, cols):
+        t = get(name)
+        if t.dim() != 2 or t.shape[1] != cols:
+            raise ValueError(f"tensor {name}: shape {tuple(t.shape)}, expected (rank, {cols})")
+        return t.to(dtype)
+
+    def vec(name, *shape):
+        t = get(name)
+        if tuple(t.shape) != tuple(shape):
+            raise ValueError(f"tensor {name}: shape {tuple(t.shape)}, expected {tuple(shape)}")
+        return t.float().contiguous().to(device)
+
+    V = cfg.vocab_size
+    w = {"embed": mat("embed", V, d).to(device), "lm_head": mat("head", V, d).to(device),
+         "final_norm": vec("final.norm", d) * cfg.logit_scale, "vocab_start": 0, "layers": [],
+         "stream_sum": torch.ones(S, dtype=torch.float32, device=device)}
+    for i, ly in enumerate(cfg.layers):
+        p, m, lw = f"l{i}.mix.", ly.mixer, LayerWeights()
+        for q in (1, 2) if ly.mlp is not None else (1,):
+            lw[f"norm{q}"] = vec(f"l{i}.norm{q}", d)
+            for n, shape in (("in", (S,)), ("out", (S,)), ("mix", (S, S))):
+                lw[f"hc{q}_{n}"] = vec(f"l{i}.hc{q}.{n}", *shape)
+        if m.kind == "parallel":
+            (a, b), (sa, sb) = m.parts, m.part_scales
+            pa, pb = p + "left.", p + "right."
+            rows_a = (("q", a.heads * a.dim), ("k", a.kv_heads * a.dim), ("v", a.kv_heads * a.vdim))
+            rows_b = (("q", b.kv_heads * b.dim), ("k", b.kv_heads * b.dim), ("v", b.heads * b.vdim))
+            a1, g1 = lowrank(pb + "a1", d), lowrank(pb + "g1", d)
+            proj, seg = _stack_segments(
+                [("left", torch.cat([mat(pa + n, r, d) for n, r in rows_a], 0), 1),
+                 ("right", torch.cat([mat(pb + n, r, d) for n, r in rows_b], 0), 1),
+                 ("b", mat(pb + "b", b.heads, d), 1), ("a1", a1, 1), ("g1", g1, 1)], d, dtype)
+            lw["proj"], lw["seg"] = proj.to(device), seg
+            lw["conv_l"] = torch.cat([vec(pa + n + ".conv", r, a.conv) for n, r in rows_a], 0).t().contiguous()
+            lw["conv_r"] = torch.cat([vec(pb + n + ".conv", r, b.conv) for n, r in rows_b], 0).contiguous()
+            lw["qn"] = vec(pa + "q.norm", a.heads * a.dim)
+            lw["kn"] = vec(pa + "k.norm", a.kv_heads * a.dim)
+            lw["a2"] = mat(pb + "a2", b.heads * b.dim, a1.shape[0]).contiguous().to(device)
+            lw["zbias"] = vec(pb + "dt_bias", b.heads * b.dim)
+            lw["rate"] = torch.exp(vec(pb + "A_log", b.heads).double()).float()
+            lw["g2"] = mat(pb + "g2", b.heads * b.vdim, g1.shape[0]).contiguous().to(device)
+            lw["gn"] = vec(pb + "norm", b.vdim) * sb
+            lw["o"] = torch.cat([mat(pa + "o", d, a.heads * a.vdim), mat(pb + "o", d, b.heads * b.vdim)],
+                                1).contiguous().to(device)
+        elif m.kind == "rope_latent_attention":
+            H, dim, rd, R, vd = m.heads, m.dim, m.rot_dim, m.kv_rank, m.vdim
+            proj, seg = _stack_segments(
+                [("qkv", torch.cat([mat(p + "q", H * (dim + rd), d), mat(p + "dkv", R + rd, d)], 0), 1),
+                 ("g", mat(p + "g", H * vd, d), 1)], d, dtype)
+            lw["proj"], lw["seg"] = proj.to(device), seg
+            lw["dkv_norm"] = vec(p + "dkv.norm", R)
+            lw["uk"] = mat(p + "uk", H * dim, R).view(H, dim, R).contiguous().to(device)
+            lw["uv_t"] = mat(p + "uv", H * vd, R).view(H, vd, R).transpose(1, 2).contiguous().to(device)
+            lw["sink"] = vec(p + "sink", H)
+            lw["o"] = mat(p + "o", d, H * vd).contiguous().to(device)
+        else:
+            raise ValueError(f"layer {i}: no weights known for mixer {m.kind!r}")
+        if ly.mlp is not None:
+            q, F = f"l{i}.mlp.", ly.mlp.ff
+            lw["gate_up"] = torch.cat([mat(q + "gate", F, d), mat(q + "up", F, d)], 0).contiguous().to(device)
+            lw["down"] = mat(q + "down", d, F).contiguous().to(device)
+        w["layers"].append(lw)
+    return w
+
+
+def init_minerax_weights(cfg, device, dtype=torch.bfloat16, seed: int = 0,
+                         keep_full: bool = True) -> dict:
+    """Seeded random Minerax weights under the checkpoint's names (tests and benchmarks):
+    projections scaled so that activations stay O(1); stream weights, convolution taps, sinks,
+    decay biases and norm weights away from their neutral values so that each shows in the logits.
+    ``keep_full`` False (benchmark sizes): drawn on the device, the name -> tensor dict is not
+    kept."""
+    d, S, full = cfg.hidden, cfg.streams, {}
+
+    def rnd(name, shape, std, mean=0.0):
+        if keep_full:
+            t = _randn(shape, std, (seed, name), "cpu", torch.float32) + mean
+            full[name] = t.to(torch.bfloat16).float()
+        else:
+            full[name] = (_randn(shape, std, (seed, name), device, torch.float32) + mean).to(torch.bfloat16)
+        return full[name]
+
+    rnd("embed", (cfg.vocab_size, d), 1.0)
+    rnd("head", (cfg.vocab_size, d), 2.0 * d ** -0.5)
+    rnd("final.norm", (d,), 0.2, 1.0)
+    for i, ly in enumerate(cfg.layers):
+        p, m = f"l{i}.mix.", ly.mixer
+        for q in (1, 2) if ly.mlp is not None else (1,):
+            rnd(f"l{i}.norm{q}", (d,), 0.2, 1.0)
+            rnd(f"l{i}.hc{q}.in", (S,), 0.3, 1.0 / S)
+            rnd(f"l{i}.hc{q}.out", (S,), 0.3, 1.0)
+            full[f"l{i}.hc{q}.mix"] = (rnd(f"l{i}.hc{q}.mix", (S, S), 0.15).float()
+                                       + 0.8 * torch.eye(S, device=full["embed"].device)
+                                       ).bfloat16().to(full["embed"].dtype)
+        if m.kind == "parallel":
+            a, b = m.parts
+            pa, pb = p + "left.", p + "right."
+            for n, r in (("q", a.heads * a.dim), ("k", a.kv_heads * a.dim), ("v", a.kv_heads * a.vdim)):
+                rnd(pa + n, (r, d), (1.0 if n == "v" else 2.0) * d ** -0.5)
+                rnd(pa + n + ".conv", (r, a.conv), 0.5)
+            rnd(pa + "q.norm", (a.heads * a.dim,), 0.2, 1.5)
+            rnd(pa + "k.norm", (a.kv_heads * a.dim,), 0.2, 1.5)
+            rnd(pa + "o", (d, a.heads * a.vdim), (a.heads * a.vdim) ** -0.5)
+            for n, r in (("q", b.kv_heads * b.dim), ("k", b.kv_heads * b.dim), ("v", b.heads * b.vdim)):
+                rnd(pb + n, (r, d), 2.0 * d ** -0.5)
+                rnd(pb + n + ".conv", (r, b.conv), 0.5)
+            rnd(pb + "b", (b.heads, d), 2.0 * d ** -0.5)
+            rnd(pb + "A_log", (b.heads,), 0.5, -1.0)
+            rnd(pb + "a1", (cfg.decay_rank, d), d ** -0.5)
+            rnd(pb + "a2", (b.heads * b.dim, cfg.decay_rank), 2.0 * cfg.decay_rank ** -0.5)
+            rnd(pb + "dt_bias", (b.heads * b.dim,), 1.0, -1.0)
+            rnd(pb + "g1", (cfg.gate_rank, d), d ** -0.5)
+            rnd(pb + "g2", (b.heads * b.vdim, cfg.gate_rank), 2.0 * cfg.gate_rank ** -0.5)
+            rnd(pb + "norm", (b.vdim,), 0.1, 1.0)
+            rnd(pb + "o", (d, b.heads * b.vdim), (b.heads * b.vdim) ** -0.5)
+        else:
+            H, dim, rd, R, vd = m.heads, m.dim, m.rot_dim, m.kv_rank, m.vdim
+            rnd(p + "q", (H * (dim + rd), d), 2.0 * d ** -0.5)
+            rnd(p + "dkv", (R + rd, d), 2.0 * d ** -0.5)
+            rnd(p + "dkv.norm", (R,), 0.1, 1.0)
+            rnd(p + "uk", (H * dim, R), 2.0 * R ** -0.5)
+            rnd(p + "uv", (H * vd, R), R ** -0.5)
+            rnd(p + "sink", (H,), 1.0)
+            rnd(p + "g", (H * vd, d), 2.0 * d ** -0.5)
+            rnd(p + "o", (d, H * vd), (H * vd) ** -0.5)
+        if ly.mlp is not None:
+            q = f"l{i}.mlp."
+            rnd(q + "gate", (ly.mlp.ff, d), d ** -0.5)
+            rnd(q + "up", (ly.mlp.ff, d), d ** -0.5)
+            rnd(q + "down", (d, ly.mlp.ff), ly.mlp.ff ** -0.5)
+    if not keep_full:
+        return _minerax_assemble(lambda k: full.pop(k), lambda k: k in full, cfg, device, dtype)
+    return minerax_from_full(full, cfg, device, dtype)
+
+
+def minerax_from_full(full: dict, cfg, device, dtype=torch.bfloat16) -> dict:
+    w = _minerax_assemble(lambda k: full[k], lambda k: k in full, cfg, device, dtype)
     w["full"] = full
     return w

@@ -1409,16 +1409,22 @@ def rotary_scaled_freq(rot_dims: int, base: float, scaling: tuple = (), device="
 def qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all: bool, k_norm_n: int, eps: float,
                           positions, inv_freq, rot_mult: float, q_rot_off: int, k_rot_off: int,
                           slot_mapping, k_cache, v_cache, H: int, G: int, qw: int, kw: int, vdim: int,
-                          v_mode: int, q_out, v_in=None, v_take: float = 0.0, v_out=None):
+                          v_mode: int, q_out, v_in=None, v_take: float = 0.0, v_out=None,
+                          neighbours: bool = False, conv=None):
+    """``conv`` = (w [taps, row width], state, row_state, row_back, row_fwd): the row's entries are
+    convolved over the sequence first."""
     if _gpu(proj):
+        cw, cs, rs, rb, rf = conv if conv is not None else (None,) * 5
         _native.mix_ops().qk_norm_rotary_append(
             proj, bias, q_norm_w, k_norm_w, bool(norm_all), int(k_norm_n), float(eps), positions,
             inv_freq, float(rot_mult), int(q_rot_off), int(k_rot_off), slot_mapping, k_cache,
-            v_cache, H, G, qw, kw, vdim, int(v_mode), q_out, v_in, float(v_take), v_out)
+            v_cache, H, G, qw, kw, vdim, int(v_mode), q_out, v_in, float(v_take), v_out,
+            bool(neighbours), cw, cs, rs, rb, rf)
     else:
         ref.qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all, k_norm_n, eps, positions,
                                   inv_freq, rot_mult, q_rot_off, k_rot_off, slot_mapping, k_cache,
-                                  v_cache, H, G, qw, kw, vdim, v_mode, q_out, v_in, v_take, v_out)
+                                  v_cache, H, G, qw, kw, vdim, v_mode, q_out, v_in, v_take, v_out,
+                                  neighbours, conv)
     return q_out
 
 
@@ -1435,22 +1441,25 @@ def keep_mfma_ok(E: int, vdim: int, block: int = 32, shared: bool = False) -> bo
 def attn_keep_window(q, k_cache, v_cache, vdim: int, block_tables, q_start, q_len, kv_len, work_seq,
                      work_qblk, head_bias, gate, out, scale: float, window: int = 0,
                      keep_first: int = 0, sigmoid: bool = False, short_rows: int = 0,
-                     mfma: bool | None = None):
+                     mfma: bool | None = None, softcap: float = 0.0, out_mult: float = 1.0):
     """Work items (sequence, block of KEEP_QBLK queries) as for attn_mixq_prefill.
     ``short_rows`` > 0: every sequence has at most that many rows (a decode section); the
     kernel then runs one workgroup per (sequence, key/value head) over one pass through the
     pages where the sizes fit its LDS.  Otherwise bf16 pages whose sizes the MFMA tiles cover
     run on them unless ``mfma`` is False (the FMA work-item kernel).  ``gate``: logits [T, H]
-    (one per head) or [T, H vdim] (one per output)."""
+    (one per head) or [T, H vdim] (one per output).  ``softcap`` > 0: softcap tanh(score / softcap);
+    the output is multiplied by ``out_mult``."""
     if _gpu(q):
         _native.mix_ops().attn_keep_window(q, k_cache, v_cache, int(vdim), block_tables, q_start,
                                            q_len, kv_len, work_seq, work_qblk, head_bias, gate, out,
                                            float(scale), int(window), int(keep_first),
                                            bool(sigmoid), int(short_rows),
-                                           KEEP_MFMA if mfma is None else bool(mfma))
+                                           KEEP_MFMA if mfma is None else bool(mfma),
+                                           float(softcap), float(out_mult))
     else:
         ref.attn_keep_window(q, k_cache, v_cache, vdim, block_tables, q_start, q_len, kv_len,
-                             head_bias, gate, out, scale, window, keep_first, sigmoid)
+                             head_bias, gate, out, scale, window, keep_first, sigmoid, softcap,
+                             out_mult)
     return out
 
 
@@ -1527,4 +1536,41 @@ def mlstm_recurrence(q, k, v, z, zbias, cap: float, q_scale: float, gate, norm_w
     else:
         ref.mlstm_recurrence(q, k, v, z, zbias, cap, q_scale, gate, norm_w, eps, S, n, m, row_state,
                              row_back, row_fwd, positions, out)
+    return out
+
+
+# ---------------------------------------------------------------------------
+# Several residual streams, a gated tanh-gelu unit, gated heads (csrc/kernels/mix_streams.hip;
+# same library).
+def streams_norm(x, y=None, mix=None, w_out=None, w_in=None, w=None, eps: float = 1e-5,
+                 centre: bool = True, out=None, keep: bool = True, ids=None, table=None):
+    """x [T, S, d] fp32, S residual streams per row: (``ids``: all of them start as the rows of
+    ``table``;) x_t <- sum_s mix[s, t] x_s + w_out[t] y (with ``y``); out = norm(sum_s w_in[s] x_s)
+    times w, a layer norm without bias (``centre``) or an RMS norm.  ``keep`` False: x is not
+    written."""
+    if _gpu(x):
+        _native.mix_ops().streams_norm(x, y, mix, w_out, w_in, w, float(eps), bool(centre), out, bool(keep),
+                                       ids, table)
+    else:
+        ref.streams_norm(x, y, mix, w_out, w_in, w, eps, centre, out, keep, ids, table)
+    return out
+
+
+def gelu_glu_rows(gate_up, out=None):
+    F = gate_up.shape[1] // 2
+    out = torch.empty((gate_up.shape[0], F), dtype=gate_up.dtype, device=gate_up.device) \
+        if out is None else out
+    if _gpu(gate_up):
+        _native.mix_ops().gelu_glu_rows(gate_up, out)
+    else:
+        ref.gelu_glu_rows(gate_up, out)
+    return out
+
+
+def gate_heads(x, gate, out):
+    """out [T, H n] = x [H, T, n] with the heads side by side, times sigmoid(gate [T, H n])."""
+    if _gpu(x):
+        _native.mix_ops().gate_heads(x, gate, out)
+    else:
+        ref.gate_heads(x, gate, out)
     return out

@@ -608,6 +608,18 @@ def conv_act_heads(x, w, state, row_state, row_back, row_fwd, positions, n_unit:
     T, C = x.shape
     if T == 0:
         return
+    y = torch.nn.functional.silu(_causal_conv(x, w, state, row_state, row_back, row_fwd, positions))
+    if n_unit > 0:
+        u = y[:, :n_unit * dim].reshape(T, n_unit, dim)
+        y[:, :n_unit * dim] = (u / torch.sqrt((u * u).sum(-1, keepdim=True) + unit_eps)).reshape(T, -1)
+    out.copy_(y)
+
+
+def _causal_conv(x, w, state, row_state, row_back, row_fwd, positions):
+    """sum_j w[:, j] x[t - (taps-1-j)] over the sequence of every row t (w [C, taps]; inputs before
+    the run from the state half [2 * slots, taps-1, C], zeros before position 0); the run's last
+    taps-1 inputs go to the other half."""
+    T, C = x.shape
     taps = w.shape[1]
     K = taps - 1
     S = state.shape[0] // 2
@@ -634,11 +646,7 @@ def conv_act_heads(x, w, state, row_state, row_back, row_fwd, positions, n_unit:
                     new[(wr, e)] = state[rd, e + n].clone()
     for (wr, e), v in new.items():
         state[wr, e] = v
-    y = torch.nn.functional.silu(acc)
-    if n_unit > 0:
-        u = y[:, :n_unit * dim].reshape(T, n_unit, dim)
-        y[:, :n_unit * dim] = (u / torch.sqrt((u * u).sum(-1, keepdim=True) + unit_eps)).reshape(T, -1)
-    out.copy_(y)
+    return acc
 
 
 def gated_linear_recurrence(q, k, v, z, rate, zbias, zsign: float, beta, gate, gate_sigmoid: bool,
@@ -745,9 +753,10 @@ def rotary_scaled_freq(rot_dims: int, base: float, scaling: tuple = (), device="
     return f.float().to(device), float(mult)
 
 
-def _rotate_halves(x, positions, inv_freq, mult: float, off: int):
-    """Entries off + i and off + i + n (n = len(inv_freq)) of the last axis of x [T, ..., w]
-    turn by the angle position * f_i; cos and sin carry the factor ``mult`` (all fp32)."""
+def _rotate_halves(x, positions, inv_freq, mult: float, off: int, neighbours: bool = False):
+    """Entries off + i and off + i + n (n = len(inv_freq)), or with ``neighbours`` off + 2i and
+    off + 2i + 1, of the last axis of x [T, ..., w] turn by the angle position * f_i; cos and sin
+    carry the factor ``mult`` (all fp32)."""
     n = inv_freq.numel()
     if n == 0:
         return x
@@ -755,29 +764,38 @@ def _rotate_halves(x, positions, inv_freq, mult: float, off: int):
     shape = (x.shape[0],) + (1,) * (x.dim() - 2) + (n,)
     c, s = (torch.cos(ang) * mult).view(shape), (torch.sin(ang) * mult).view(shape)
     y = x.clone()
-    u, v = x[..., off:off + n], x[..., off + n:off + 2 * n]
-    y[..., off:off + n] = u * c - v * s
-    y[..., off + n:off + 2 * n] = v * c + u * s
+    first = slice(off, off + 2 * n, 2) if neighbours else slice(off, off + n)
+    second = slice(off + 1, off + 2 * n, 2) if neighbours else slice(off + n, off + 2 * n)
+    u, v = x[..., first], x[..., second]
+    y[..., first] = u * c - v * s
+    y[..., second] = v * c + u * s
     return y
 
 
 def qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all: bool, k_norm_n: int, eps: float,
                           positions, inv_freq, rot_mult: float, q_rot_off: int, k_rot_off: int,
                           slot_mapping, k_cache, v_cache, H: int, G: int, qw: int, kw: int, vdim: int,
-                          v_mode: int, q_out, v_in=None, v_take: float = 0.0, v_out=None) -> None:
+                          v_mode: int, q_out, v_in=None, v_take: float = 0.0, v_out=None,
+                          neighbours: bool = False, conv=None) -> None:
     """Rows of proj are q [H, qw] | k [G, kw] (| v [G, vdim] with v_mode 0); ``bias`` (fp32, the
     row's width) is added first.  RMS norms with plain weights: over the whole q and the whole k
     projection (``norm_all``; weights [H qw], [G kw]) or per head, q over its qw entries
     (weight [qw]) and k over its leading ``k_norm_n`` entries (weight [k_norm_n]); a weight of
-    None means no norm.  Then the half-split rotation of entries rot_off .. rot_off + 2 n of
-    every head.  q goes to q_out [T, H, qw] fp32; k rows into k_cache [blocks, G, BS, kw];
+    None means no norm.  Then the half-split rotation (``neighbours``: in pairs of neighbouring
+    entries) of entries rot_off .. rot_off + 2 n of every head.  q goes to q_out [T, H, qw] fp32; k rows into k_cache [blocks, G, BS, kw];
     values into v_cache [blocks, G, BS, vdim]: v_mode 0 the v columns, 1 the keys as projected
     (before norm and rotation), 2 none.  ``v_out`` [T, G vdim] fp32 receives the values as
-    projected; with ``v_in`` [T, G vdim] fp32 the cached ones are (1 - v_take) v + v_take v_in."""
+    projected; with ``v_in`` [T, G vdim] fp32 the cached ones are (1 - v_take) v + v_take v_in.
+    ``conv`` = (w [taps, row width] fp32, state [2 * slots, taps - 1, row width], row_state,
+    row_back, row_fwd): before everything else each entry becomes its causal convolution over
+    the sequence's rows."""
     T = proj.shape[0]
     if T == 0:
         return
     x = proj.float()
+    if conv is not None:
+        w, state, row_state, row_back, row_fwd = conv
+        x = _causal_conv(x[:, :w.shape[1]], w.float().t(), state, row_state, row_back, row_fwd, positions)
     if bias is not None:
         x = x[:, :bias.numel()] + bias.float()
     nq, nk = H * qw, G * kw
@@ -795,8 +813,8 @@ def qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all: bool, k_norm
             q = _rms(q, eps) * q_norm_w.float()
         if k_norm_w is not None:
             k[..., :k_norm_n] = _rms(k[..., :k_norm_n], eps) * k_norm_w.float()
-    q = _rotate_halves(q, positions[:T], inv_freq, rot_mult, q_rot_off)
-    k = _rotate_halves(k, positions[:T], inv_freq, rot_mult, k_rot_off)
+    q = _rotate_halves(q, positions[:T], inv_freq, rot_mult, q_rot_off, neighbours)
+    k = _rotate_halves(k, positions[:T], inv_freq, rot_mult, k_rot_off, neighbours)
     q_out.copy_(q)
     if k_cache is None or G == 0:
         return
@@ -815,14 +833,16 @@ def qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all: bool, k_norm
 
 
 def attn_keep_window(q, k_cache, v_cache, vdim: int, block_tables, q_start, q_len, kv_len, head_bias,
-                     gate, out, scale: float, window: int, keep_first: int, sigmoid: bool) -> None:
+                     gate, out, scale: float, window: int, keep_first: int, sigmoid: bool,
+                     softcap: float = 0.0, out_mult: float = 1.0) -> None:
     """q [T, H, E] fp32; k_cache [blocks, G, BS, E]; the values are the first ``vdim`` entries
     of v_cache's rows (which may be the key pages themselves).  Position i sees j <= i with
     i - j < window or j < keep_first (window 0: every j <= i).  Weights: softmax over the
     visible keys, with exp(head_bias[h]) added to the denominator when head_bias is given; or
     (``sigmoid``) sigmoid(score + head_bias[h]) per visible key, not normalised.  ``gate``
     [T, H] (one logit per head) or [T, H vdim] (one per output): the output is multiplied by
-    sigmoid(gate).  out [T, H vdim]."""
+    sigmoid(gate), and in any case by out_mult.  softcap > 0: scores (scaled) become
+    softcap tanh(score / softcap).  out [T, H vdim]."""
     H = q.shape[1]
     G = k_cache.shape[1]
     rep = H // G
@@ -838,6 +858,8 @@ def attn_keep_window(q, k_cache, v_cache, vdim: int, block_tables, q_start, q_le
         if window > 0:
             ok = ok & ((i - j < window) | (j < keep_first))
         s = torch.einsum("qhe,hke->hqk", q[t0:t0 + ql].float(), k) * scale
+        if softcap > 0:
+            s = softcap * torch.tanh(s / softcap)
         if sigmoid:
             p = torch.sigmoid(s + head_bias.float()[:, None, None]) * ok[None]
         else:
@@ -845,7 +867,7 @@ def attn_keep_window(q, k_cache, v_cache, vdim: int, block_tables, q_start, q_le
             if head_bias is not None:
                 s = torch.cat([s, head_bias.float()[:, None, None].expand(H, ql, 1)], -1)
             p = torch.softmax(s, -1)[..., :kl]
-        o = torch.einsum("hqk,hkd->qhd", p, v)
+        o = torch.einsum("hqk,hkd->qhd", p, v) * out_mult
         if gate is not None:
             o = o * torch.sigmoid(gate[t0:t0 + ql].float()).reshape(ql, H, -1)
         out[t0:t0 + ql].copy_(o.reshape(ql, -1).to(out.dtype))
@@ -952,3 +974,34 @@ def mlstm_recurrence(q, k, v, z, zbias, cap: float, q_scale: float, gate, norm_w
             S[wr], n[wr], m[wr] = cs, cn, cm
     y = _rms(o, eps) * norm_w.float().view(H, vdim) * torch.sigmoid(gate.float().reshape(T, H, vdim))
     out.copy_(y.reshape(T, H * vdim).to(out.dtype))
+
+
+# ---------------------------------------------------------------------------
+# Several residual streams, a gated tanh-gelu unit, gated heads.
+def streams_norm(x, y, mix, w_out, w_in, w, eps: float, centre: bool, out, keep: bool, ids, table) -> None:
+    """x [T, S, d] fp32 holds S residual streams of every row.  With ``ids`` they all start as the
+    rows of ``table``.  With ``y`` [T, d]: x_t <- sum_s mix[s, t] x_s + w_out[t] y, all streams from
+    the old ones.  u = sum_s w_in[s] x_s; out = w u / sqrt(mean(u^2) + eps), ``centre``: with
+    u less its mean (a layer norm without bias).  ``keep`` False: x need not be written (nobody
+    reads it afterwards)."""
+    if ids is not None:
+        x.copy_(table[ids.long()].float()[:, None].expand_as(x))
+    if y is not None:
+        x.copy_(torch.einsum("tsd,su->tud", x, mix.float()) + w_out.float()[None, :, None] * y.float()[:, None])
+    u = torch.einsum("tsd,s->td", x, w_in.float())
+    if centre:
+        u = u - u.mean(-1, keepdim=True)
+    out.copy_((_rms(u, eps) * w.float()).to(out.dtype))
+
+
+def gelu_glu_rows(gate_up, out) -> None:
+    """out = g(gate) * up of rows [gate | up], g(z) = z/2 (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))."""
+    F = gate_up.shape[1] // 2
+    g = torch.nn.functional.gelu(gate_up[:, :F].float(), approximate="tanh")
+    out.copy_((g * gate_up[:, F:].float()).to(out.dtype))
+
+
+def gate_heads(x, gate, out) -> None:
+    """x [H, T, n] -> out [T, H n] = x * sigmoid(gate), gate [T, H n] logits."""
+    H, T, n = x.shape
+    out.copy_((x.float().transpose(0, 1).reshape(T, H * n) * torch.sigmoid(gate.float())).to(out.dtype))
