@@ -77,9 +77,9 @@ def parse():
     ap.add_argument("--arch-sizes", default="", help="--arch-compare: size classes, comma separated")
     ap.add_argument("--arch-models", default="",
                     help="--arch-compare: which of the two models to run (default both), comma separated; "
-                         "'kernels' (bilolix, nutitar, modepel): only the per-kernel times")
+                         "'kernels' (bilolix, nutitar, modepel, minerax): only the per-kernel times")
     ap.add_argument("--arch-compare", default="",
-                    help="livisun | numalorn | bilolix | nutitar | modepel: instead of the RFQ workload, time prefill and decode "
+                    help="livisun | numalorn | bilolix | nutitar | modepel | minerax: instead of the RFQ workload, time prefill and decode "
                          "of the layer-list model beside the closest decoder at equal layer sizes "
                          "(replisense_rfq_amd/benchmarks/arch_compare.py); one JSON line")
     ap.add_argument("--time-budget", type=float, default=0.0,
@@ -368,8 +368,9 @@ def main():
     t_start = time.perf_counter()
     if args.arch_compare:
         if args.arch_compare not in ("livisun", "numalorn", "bilolix", "nutitar",
-                                     "modepel") or args.gpus != 1:
-            raise SystemExit("bench: --arch-compare livisun | numalorn | bilolix | nutitar | modepel runs on one GPU")
+                                     "modepel", "minerax") or args.gpus != 1:
+            raise SystemExit("bench: --arch-compare livisun | numalorn | bilolix | nutitar | modepel | minerax "
+                             "runs on one GPU")
         from replisense_rfq_amd.benchmarks import arch_compare
 
         extra = {}
@@ -390,6 +391,10 @@ def main():
             from replisense_rfq_amd.benchmarks import arch_kernels
 
             extra["kernels"] = arch_kernels.run_modepel(args)
+        if args.arch_compare == "minerax" and (not args.arch_models or "kernels" in args.arch_models):
+            from replisense_rfq_amd.benchmarks import arch_kernels
+
+            extra["kernels"] = arch_kernels.run_minerax(args)
         print(json.dumps({"metric": "arch_compare", "arch": args.arch_compare, "dtype": "bf16",
                           "data": "synthetic", **arch_compare.run(args), **extra}), flush=True)
         return

@@ -74,7 +74,7 @@ bool launch_qk_norm_rotary_append(bool, const void*, int64_t, const float*, cons
                                   const float*, bool, int, float, const int32_t*, const float*, int,
                                   float, int, int, const int32_t*, void*, void*, int, int, int, int,
                                   int, int, int, int, int64_t, const float*, float, float*, float*,
-                                  bool, const float*, int, float*, int, const int32_t*,
+                                  int64_t, int64_t, int, bool, const float*, int, float*, int, const int32_t*,
                                   const int32_t*, const int32_t*, hipStream_t);
 bool launch_attn_keep_window(bool, const float*, const void*, const void*, int64_t, const int32_t*,
                              int, const int32_t*, const int32_t*, const int32_t*, const int32_t*,
@@ -685,8 +685,16 @@ void qk_norm_rotary_append(const Tensor& proj, const OptT& bias, const OptT& q_n
   const int64_t W = H * qw + G * kw + (v_mode == 0 ? G * vdim : 0);
   TORCH_CHECK(proj.size(1) >= W, "qk_norm_rotary_append: proj narrower than q | k | v");
   TORCH_CHECK(v_mode != 1 || vdim == kw, "qk_norm_rotary_append: values that are the keys have their width");
+  // q_out may be a slice of wider rows, and may hold only the trailing entries of every head (which
+  // are then all of q that is read)
+  TORCH_CHECK(q_out.is_cuda() && q_out.scalar_type() == at::kFloat && q_out.dim() == 3 && q_out.size(0) == T &&
+              q_out.size(1) == H && q_out.size(2) >= 1 && q_out.size(2) <= qw && q_out.stride(2) == 1,
+              "qk_norm_rotary_append: q_out [T, H, <= qw] float32");
+  const int64_t qn = q_out.size(2), q_from = qw - qn;
+  TORCH_CHECK(q_from == 0 || (!q_norm_w.has_value() && !bias.has_value() && !conv_w.has_value() && !norm_all),
+              "qk_norm_rotary_append: trailing entries of q come without norm, bias and convolution");
   const int nrot = (int)inv_freq.numel();
-  TORCH_CHECK(q_rot_off >= 0 && k_rot_off >= 0 && q_rot_off + 2 * nrot <= qw &&
+  TORCH_CHECK(q_rot_off >= q_from && k_rot_off >= 0 && q_rot_off + 2 * nrot <= qw &&
               (G == 0 || k_rot_off + 2 * nrot <= kw),
               "qk_norm_rotary_append: the rotated entries lie outside a head");
   TORCH_CHECK(k_norm_n >= 0 && k_norm_n <= kw && (!norm_all || k_norm_n == kw),
@@ -714,8 +722,6 @@ void qk_norm_rotary_append(const Tensor& proj, const OptT& bias, const OptT& q_n
       vp = vc.data_ptr();
     }
   }
-  TORCH_CHECK(q_out.dim() == 3 && q_out.size(0) == T && q_out.size(1) == H && q_out.size(2) == qw,
-              "qk_norm_rotary_append: q_out [T, H, qw]");
   TORCH_CHECK((!v_in.has_value() && !v_out.has_value()) || (v_mode != 2 && G > 0),
               "qk_norm_rotary_append: blended values need values");
   const int64_t nv = (int64_t)T * G * vdim;
@@ -741,10 +747,10 @@ void qk_norm_rotary_append(const Tensor& proj, const OptT& bias, const OptT& q_n
       f32, proj.data_ptr(), proj.stride(0), optf(bias, "bias", W), optf(q_norm_w, "q_norm_w", nqw),
       (G > 0 && k_norm_w.has_value()) ? f32p(*k_norm_w, "k_norm_w", nkw) : nullptr, norm_all,
       (int)k_norm_n, (float)eps, i32p(pos, "positions", T), fr, nrot, (float)rot_mult,
-      (int)q_rot_off, (int)k_rot_off, i32p(slots, "slots", T), kp, vp, T, (int)H, (int)G, (int)qw,
+      (int)(q_rot_off - q_from), (int)k_rot_off, i32p(slots, "slots", T), kp, vp, T, (int)H, (int)G, (int)qn,
       (int)kw, (int)vdim, (int)v_mode, BS, pool_slots, optf(v_in, "v_in", nv), (float)v_take,
-      const_cast<float*>(optf(v_out, "v_out", nv)), const_cast<float*>(f32p(q_out, "q_out")),
-      neighbours, taps > 0 ? f32p(*conv_w, "conv_w") : nullptr, taps, cst, state_slots, rs, rb, rf,
+      const_cast<float*>(optf(v_out, "v_out", nv)), q_out.data_ptr<float>(), q_out.stride(0),
+      q_out.stride(1), (int)q_from, neighbours, taps > 0 ? f32p(*conv_w, "conv_w") : nullptr, taps, cst, state_slots, rs, rb, rf,
       stream());
   TORCH_CHECK(ok, "qk_norm_rotary_append: a row does not fit the LDS");
 }

@@ -4,7 +4,8 @@
 //   qk_norm_rotary_append   rows q [H, qw] | k [G, kw] (| v [G, vdim]) of a fused projection:
 //                           bias, causal convolution over the sequence's rows, RMS norm per head or
 //                           over the whole projection, rotation of entries (off + i, off + i + n) or
-//                           (off + 2i, off + 2i + 1) by pos * f_i with a factor on cos and sin; q out in fp32, k and the values into their page rows; the
+//                           (off + 2i, off + 2i + 1) by pos * f_i with a factor on cos and sin
+//                           (q may consist of the entries from q_from on of wider heads); q out in fp32, k and the values into their page rows; the
 //                           values may be blended with another layer's values of the same token
 //                           (v <- keep v + take v_in) and handed on unblended (v_out)
 //   attn_keep_window        s(i, j) = scale q_h(i) . k_g(j);  i sees j <= i with
@@ -95,6 +96,8 @@ __device__ __forceinline__ void st_chunk(bf16_t* p, const float* f) {
 // conv_w [taps][W]: the row is first convolved over the rows of its sequence (rows before the run
 // come from the state half that row_state names, zeros before position 0; the run's last taps - 1
 // rows go to the other half).
+// q_from > 0 (no convolution): a head of q holds q_from + qw entries in proj, of which only the
+// last qw are read; everything below sees heads of qw entries.
 // LDS (floats): row[W] | fac[H + G] | cs[2 nrot] | scratch[16]
 template <typename T, int CW>
 __global__ __launch_bounds__(256) void qk_norm_rotary_append_kernel(
@@ -104,9 +107,9 @@ __global__ __launch_bounds__(256) void qk_norm_rotary_append_kernel(
     int nrot, float rot_mult, int q_rot_off, int k_rot_off, const int32_t* __restrict__ slots,
     T* __restrict__ k_cache, T* __restrict__ v_cache, int H, int G, int qw, int kw, int vdim,
     int v_mode, int BS, int64_t pool_slots, const float* __restrict__ v_in, float v_keep,
-    float v_take, float* __restrict__ v_out, float* __restrict__ q_out, int neighbours,
-    const float* __restrict__ conv_w, int taps, float* __restrict__ conv_state, int state_slots,
-    const int32_t* __restrict__ row_state, const int32_t* __restrict__ row_back,
+    float v_take, float* __restrict__ v_out, float* __restrict__ q_out, int64_t q_ts,
+    int64_t q_hs, int q_from, int neighbours, const float* __restrict__ conv_w, int taps,
+    float* __restrict__ conv_state, int state_slots, const int32_t* __restrict__ row_state, const int32_t* __restrict__ row_back,
     const int32_t* __restrict__ row_fwd) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int t = blockIdx.x, tid = threadIdx.x, nthr = blockDim.x;
@@ -135,9 +138,11 @@ __global__ __launch_bounds__(256) void qk_norm_rotary_append_kernel(
       wr = conv_state + ((int64_t)((1 - (code & 1)) * state_slots + (code >> 1)) * K) * W;
     }
   }
+  const T* src_k = src + H * q_from;   // entries behind q
   for (int c = tid * CW; c < W; c += nthr * CW) {
     float f[CW];
-    ld_chunk<CW>(src + c, f);
+    if (q_from > 0 && c < nq) ld_chunk<CW>(src + (c / qw + 1) * q_from + c, f);
+    else ld_chunk<CW>(src_k + c, f);
     if (conv_w != nullptr) {
       float u[CW], w[CW];
       if (wr != nullptr) {
@@ -314,7 +319,7 @@ __global__ __launch_bounds__(256) void qk_norm_rotary_append_kernel(
       }
     }
     if (isq)
-      st_chunk<CW>(q_out + (int64_t)t * nq + c, v);
+      st_chunk<CW>(q_out + t * q_ts + hd * q_hs + e, v);
     else if (keep)
       st_chunk<CW>(k_cache + (page_row + (int64_t)hd * BS) * kw + e, v);
   }
@@ -706,7 +711,8 @@ bool launch_qk_norm_rotary_append(bool f32, const void* proj, int64_t stride, co
                                   int k_rot_off, const int32_t* slots, void* k_cache, void* v_cache,
                                   int T, int H, int G, int qw, int kw, int vdim, int v_mode, int BS,
                                   int64_t pool_slots, const float* v_in, float v_take,
-                                  float* v_out, float* q_out, bool neighbours, const float* conv_w,
+                                  float* v_out, float* q_out, int64_t q_ts, int64_t q_hs, int q_from,
+                                  bool neighbours, const float* conv_w,
                                   int taps, float* conv_state, int state_slots,
                                   const int32_t* row_state, const int32_t* row_back,
                                   const int32_t* row_fwd, hipStream_t s) {
@@ -727,13 +733,15 @@ bool launch_qk_norm_rotary_append(bool f32, const void* proj, int64_t stride, co
                    stride % 8 == 0 && k_norm_n % 8 == 0 && nrot % 8 == 0 && q_rot_off % 8 == 0 &&
                    k_rot_off % 8 == 0 && al16(proj) && al16(bias) && al16(q_norm_w) &&
                    al16(k_norm_w) && al16(k_cache) && al16(v_cache) && al16(q_out) && al16(v_in) &&
-                   al16(v_out) && al16(conv_w) && al16(conv_state);
+                   al16(v_out) && al16(conv_w) && al16(conv_state) && q_ts % 8 == 0 && q_hs % 8 == 0 &&
+                   q_from % 8 == 0;
 #define QKN_GO(TT, CW)                                                                          \
   hipLaunchKernelGGL((qk_norm_rotary_append_kernel<TT, CW>), dim3(T), dim3(256), lds, s,       \
                      (const TT*)proj, stride, bias, q_norm_w, k_norm_w, (int)norm_all, k_norm_n, \
                      eps, pos, inv_freq, nrot, rot_mult, q_rot_off, k_rot_off, slots,           \
                      (TT*)k_cache, (TT*)v_cache, H, G, qw, kw, vdim, v_mode, BS, pool_slots,    \
-                     v_in, 1.0f - v_take, v_take, v_out, q_out, (int)neighbours, conv_w, taps,  \
+                     v_in, 1.0f - v_take, v_take, v_out, q_out, q_ts, q_hs, q_from,             \
+                     (int)neighbours, conv_w, taps,                                             \
                      conv_state, state_slots, row_state, row_back, row_fwd)
   if (f32) {
     if (vec) QKN_GO(float, 8);

@@ -297,8 +297,8 @@ __global__ __launch_bounds__(128 * HPW) void attn_keep_mfma_kernel(
 namespace {
 bool plain_sizes(int DK, int DV) { return DK >= 1 && DK <= 4 && (DV == 2 || DV == 4 || DV == 8); }
 bool shared_sizes(int DK, int DV) {
-  return (DK == 3 && DV == 4) || (DK == 5 && DV == 8) || (DK == 6 && DV == 8) ||
-         (DK == 10 && DV == 16) || (DK == 18 && DV == 32);
+  return (DK == 3 && DV == 4) || (DK == 4 && (DV == 4 || DV == 6)) || (DK == 5 && DV == 8) ||
+         (DK == 6 && DV == 8) || (DK == 10 && DV == 16) || (DK == 18 && DV == 32);
 }
 }  // namespace
 
@@ -377,6 +377,8 @@ bool launch_attn_keep_mfma(const float* q, const void* k_cache, const void* v_ca
   const int DK = E / 32, DV = vdim / 16;
   if (shared) {
     if (DK == 3) launch_keep_mfma_heads<3, 4, true>(a);
+    else if (DK == 4 && DV == 4) launch_keep_mfma_heads<4, 4, true>(a);
+    else if (DK == 4) launch_keep_mfma_heads<4, 6, true>(a);
     else if (DK == 5) launch_keep_mfma_heads<5, 8, true>(a);
     else if (DK == 6) launch_keep_mfma_heads<6, 8, true>(a);
     else if (DK == 10) launch_keep_mfma_heads<10, 16, true>(a);

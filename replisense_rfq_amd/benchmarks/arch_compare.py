@@ -4,8 +4,10 @@ framework at equal layer sizes: ``bench.py --arch-compare livisun`` (beside Llam
 experts, choices per token and expert width), ``--arch-compare bilolix`` (beside Numalorn:
 same width, head count, experts and expert width; attention and recurrent layers alternate
 in both), ``--arch-compare nutitar`` (beside Bilolix with attention in every layer: same
-width, head counts and dense feed-forward width) and ``--arch-compare modepel`` (beside Bilolix:
-attention and recurrent layers alternate in both, the same experts in every layer).
+width, head counts and dense feed-forward width), ``--arch-compare modepel`` (beside Bilolix:
+attention and recurrent layers alternate in both, the same experts in every layer) and
+``--arch-compare minerax`` (beside Bilolix with attention and delta-rule layers, and beside
+Nutitar with latent layers; feed-forwards of equal weights).
 
 Both run through the same engine (scheduler, paged cache, hipGraph decode steps), with
 random weights, a few layers of a real model's shape and a small vocabulary, so the numbers
@@ -132,6 +134,34 @@ def _modepel_configs(name, d, H, G, *ff):
     return bil, mod
 
 
+def _minerax_configs(name, d, H, G, F):
+    """Bilolix, Nutitar and Minerax at equal sizes; the two-matrix feed-forwards are 3 F / 2 wide,
+    so that they hold as many weights as Minerax's three matrices.  Bilolix: attention (two 64-wide
+    maps per head, 128-wide values, no window) alternating with the delta rule on d/128 heads with
+    64 x 128 states.  Nutitar: latent attention in every layer (128 plain + 64 rotated query
+    dimensions per head over a 512-wide latent of each layer's own, no window).  Minerax: two layers
+    that hold such an attention (128-wide heads) AND such a delta rule side by side, alternating
+    with two such latent layers (window 1,024); two residual streams."""
+    from ..models.config import bilolix_layers, minerax_layers, nutitar_layers
+
+    bil = LayeredConfig(f"cmp-bilolix-{name}", architecture="Bilolix", vocab_size=VOCAB, hidden=d,
+                        canon_taps=0, decay_rank=64, gate_rank=64, loop=(0, 0, 1),
+                        layers=bilolix_layers("acac"[:LAYERS], H, G, 64, 128, 3 * F // 2, window=0,
+                                              rot_dims=64, rot_base=5e5, rec_heads=d // 128, rec_dim=64))
+    nut = LayeredConfig(f"cmp-nutitar-{name}", architecture="Nutitar", vocab_size=VOCAB, hidden=d,
+                        canon_taps=0, embed_scale=1.0, residual_mult=0.5, token_shift=True,
+                        layers=nutitar_layers("llll"[:LAYERS], H, G, 128, 128, 3 * F // 2, kv_rank=512,
+                                              rot_dim=64, rot_dims=64, rot_base=5e5,
+                                              yarn=(4.0, 4096.0, 32.0, 1.0)))
+    mnx = LayeredConfig(f"cmp-minerax-{name}", architecture="Minerax", vocab_size=VOCAB, hidden=d,
+                        canon_taps=0, decay_rank=64, gate_rank=64, streams=2,
+                        layers=minerax_layers("plpl"[:LAYERS], H, G, 128, 128, F, conv=4, softcap=30.0,
+                                              rec_heads=d // 128, rec_dim=64, kv_rank=512, rot_dim=64,
+                                              window=1024, rot_dims=64, rot_base=5e5,
+                                              yarn=(4.0, 4096.0, 32.0, 1.0)))
+    return bil, nut, mnx
+
+
 def _engine(mcfg, args, batch):
     from ..models import layered_model_class
     from ..models.llama import DecoderLM
@@ -160,6 +190,11 @@ def _engine(mcfg, args, batch):
             # choices spread over all outputs, as a trained correction keeps them
             if "correction" in lw:
                 lw["correction"].mul_(0.05)
+        model = layered_model_class(mcfg.architecture)(mcfg, dev, weights=w)
+    elif isinstance(mcfg, LayeredConfig) and mcfg.architecture == "Minerax":
+        from ..models.weights import init_minerax_weights
+
+        w = init_minerax_weights(mcfg, dev, torch.bfloat16, args.seed, keep_full=False)
         model = layered_model_class(mcfg.architecture)(mcfg, dev, weights=w)
     elif isinstance(mcfg, LayeredConfig):
         model = layered_model_class(mcfg.architecture)(mcfg, dev, seed=args.seed)
@@ -202,11 +237,12 @@ def run(args) -> dict:
     only = [x for x in getattr(args, "arch_sizes", "").split(",") if x]
     arch = getattr(args, "arch_compare", "livisun")
     base = {"livisun": "llama", "numalorn": "sparse", "bilolix": "numalorn", "nutitar": "bilolix",
-            "modepel": "bilolix"}[arch]
+            "modepel": "bilolix", "minerax": "bilolix"}[arch]
     make = {"livisun": _configs, "numalorn": _moe_configs, "bilolix": _bilolix_configs,
-            "nutitar": _nutitar_configs, "modepel": _modepel_configs}[arch]
+            "nutitar": _nutitar_configs, "modepel": _modepel_configs,
+            "minerax": _minerax_configs}[arch]
     sizes = SIZES[:2] + MOE_SIZES if arch == "modepel" else \
-        SIZES if arch in ("livisun", "nutitar") else MOE_SIZES
+        SIZES if arch in ("livisun", "nutitar", "minerax") else MOE_SIZES
     for size in sizes:
         name = size[0]
         if only and name not in only:
@@ -234,6 +270,9 @@ def run(args) -> dict:
         if arch in row and base in row:
             row["prefill_ratio"] = round(row[arch]["prefill_tok_s"] / row[base]["prefill_tok_s"], 3)
             row["decode_ratio"] = round(row[arch]["decode_tok_s"] / row[base]["decode_tok_s"], 3)
+        if arch == "minerax" and arch in row and "nutitar" in row:
+            row["prefill_ratio_nutitar"] = round(row[arch]["prefill_tok_s"] / row["nutitar"]["prefill_tok_s"], 3)
+            row["decode_ratio_nutitar"] = round(row[arch]["decode_tok_s"] / row["nutitar"]["decode_tok_s"], 3)
         out["sizes"][name] = row
     return out
 

@@ -537,3 +537,128 @@ def run_modepel(args) -> dict:
         _experts(T, d, 14336, 8, 2, like)
         res[key] = {"modepel": mine, "like": like}
     return res
+
+
+# ---------------------------------------------------------------------------
+# Minerax's kernels (``bench.py --arch-compare minerax``) beside the like kernels of Bilolix,
+# Nutitar and Modepel in the same run: 4096-wide layers with two residual streams, 32 heads over
+# 8 key/value heads of 128, 32 recurrent heads with 64 x 128 states, a 512-wide latent with a
+# 64-wide rotated key part inside a window of 1,024.
+def _x_rows(T, d, out):
+    g = torch.Generator(device=DEV).manual_seed(0)
+    S = 2
+    x = torch.randn(T, S, d, generator=g, device=DEV)
+    y = torch.randn(T, d, generator=g, device=DEV).bfloat16()
+    h = torch.empty(T, d, dtype=torch.bfloat16, device=DEV)
+    mix = torch.eye(S, device=DEV) * 0.7 + 0.15
+    wo, wi = torch.ones(S, device=DEV) * 0.01, torch.ones(S, device=DEV)
+    w = torch.ones(d, device=DEV)
+    out["streams_norm"] = _entry(_time(lambda: ops.streams_norm(x, y, mix, wo, wi, w, 1e-5, out=h)),
+                                 T * d * (8 * S + 4), 0)
+    F = 14336
+    u = torch.randn(T, 2 * F, generator=g, device=DEV).bfloat16()
+    o = torch.empty(T, F, dtype=torch.bfloat16, device=DEV)
+    out["gelu_glu_rows"] = _entry(_time(lambda: ops.gelu_glu_rows(u, o)), T * F * 6, 0)
+    H, n = 32, 128
+    a = torch.randn(H, T, n, generator=g, device=DEV).bfloat16()
+    gt = torch.randn(T, H * n, generator=g, device=DEV).bfloat16()
+    b = torch.empty(T, H * n, dtype=torch.bfloat16, device=DEV)
+    out["gate_heads"] = _entry(_time(lambda: ops.gate_heads(a, gt, b)), T * H * n * 6, 0)
+
+
+def _x_attention(H, G, dim, lens, q_lens, rows, out, name):
+    """Left mixer: convolution, norms over the projections and rotation in one kernel, softcapped
+    attention.  ``rows``: the runs' places."""
+    g = torch.Generator(device=DEV).manual_seed(3)
+    T = sum(q_lens)
+    kc, vc, pos, sl, meta = _pages(lens, q_lens, G, dim, dim, g)
+    n = (H + 2 * G) * dim
+    pr = (torch.randn(T, n, generator=g, device=DEV) * 0.5).bfloat16()
+    taps = 4
+    cw = torch.randn(taps, n, generator=g, device=DEV) * 0.5
+    cst = torch.zeros(128, taps - 1, n, device=DEV)
+    qn, kn = torch.randn(H * dim, generator=g, device=DEV), torch.randn(G * dim, generator=g, device=DEV)
+    inv, mult = ops.rotary_scaled_freq(64, 5e5, ("yarn", 4.0, 4096.0, 32.0, 1.0), DEV)
+    q = torch.empty(T, H, dim, device=DEV)
+    rs, rb, rf, _ = rows
+    t = _time(lambda: ops.qk_norm_rotary_append(pr, None, qn, kn, True, dim, 1e-5, pos, inv, mult, 0, 0, sl, kc,
+                                                vc, H, G, dim, dim, dim, 0, q, conv=(cw, cst, rs, rb, rf)))
+    state = len(lens) * (taps - 1) * n * (8 if name == "decode" else 4)
+    out[f"qk_norm_rotary_append conv ({name})"] = _entry(
+        t, T * n * 2 + T * H * dim * 4 + T * G * 2 * dim * 2 + state, 0)
+    o = torch.empty(T, H * dim, dtype=torch.bfloat16, device=DEV)
+    pairs = sum(p + 1 for n_, q_ in zip(lens, q_lens) for p in range(n_ - q_, n_))
+    nbytes = sum(lens) * G * 2 * dim * 2 + T * H * dim * 6
+    bt, qs, ql, kl, ws, wq = meta
+    short = ops.TALK_DECODE_MAX_ROWS if name == "decode" else 0
+    t = _time(lambda: ops.attn_keep_window(q, kc, vc, dim, bt, qs, ql, kl, ws, wq, None, None, o, dim ** -0.5,
+                                           short_rows=short, softcap=30.0, out_mult=0.6), reps=5, warm=2)
+    out[f"attn_keep_window softcap ({name})"] = _entry(t, nbytes, 4.0 * dim * H * pairs)
+
+
+def _x_latent(H, lens, q_lens, window, out, name):
+    """Latent layer: queries carried into the latent space, norm and rotation, windowed
+    attention, W_uv and the gate."""
+    g = torch.Generator(device=DEV).manual_seed(3)
+    T = sum(q_lens)
+    dim, R, rd, vd = 128, 512, 64, 128
+    E = R + rd
+    kc, _, pos, sl, meta = _pages(lens, q_lens, 1, E, 0, g)
+    nq = H * (dim + rd)
+    pr = (torch.randn(T, nq + E, generator=g, device=DEV) * 0.5).bfloat16()
+    nw = torch.randn(R, generator=g, device=DEV)
+    uk = (torch.randn(H, dim, R, generator=g, device=DEV) * R ** -0.5).bfloat16()
+    uv = (torch.randn(H, R, vd, generator=g, device=DEV) * R ** -0.5).bfloat16()
+    inv, mult = ops.rotary_scaled_freq(rd, 5e5, ("yarn", 4.0, 4096.0, 32.0, 1.0), DEV)
+    q = torch.empty(T, H, E, device=DEV)
+    t = _time(lambda: ops.qk_norm_rotary_append(pr, None, None, nw, False, R, 1e-5, pos, inv, mult, dim, R, sl,
+                                                kc, None, H, 1, dim + rd, E, 0, 2, q[:, :, R:], neighbours=True))
+    out[f"qk_norm_rotary_append latent ({name})"] = _entry(
+        t, T * (H * rd + E) * 2 + T * H * rd * 4 + T * E * 2, 0)
+    qn = pr[:, :nq].unflatten(1, (H, dim + rd))[:, :, :dim].transpose(0, 1)
+    t = _time(lambda: ops.bmm_f32(qn, uk, out=q[:, :, :R].transpose(0, 1)))
+    out[f"latent queries, vendor product ({name})"] = _entry(t, T * H * (dim * 2 + R * 4), 2.0 * T * H * dim * R)
+    q.normal_(generator=g).mul_(0.3)
+    sink = torch.randn(H, generator=g, device=DEV)
+    lat = torch.empty(T, H * R, dtype=torch.bfloat16, device=DEV)
+    pairs = seen = 0
+    for n_, q_ in zip(lens, q_lens):
+        pairs += sum(min(p + 1, window) if window else p + 1 for p in range(n_ - q_, n_))
+        seen += min(n_, window + q_ - 1) if window else n_
+    bt, qs, ql, kl, ws, wq = meta
+    short = ops.TALK_DECODE_MAX_ROWS if name == "decode" else 0
+    t = _time(lambda: ops.attn_keep_window(q, kc, kc, R, bt, qs, ql, kl, ws, wq, sink, None, lat, E ** -0.5,
+                                           window, short_rows=short), reps=5, warm=2)
+    out[f"attn_keep_window latent ({name})"] = _entry(
+        t, seen * E * 2 + T * H * (E * 4 + R * 2), (2.0 * E + 2.0 * R) * H * pairs)
+    t = _time(lambda: torch.bmm(lat.view(T, H, R).transpose(0, 1), uv))
+    out[f"latent values, vendor product ({name})"] = _entry(t, T * H * (R + vd) * 2, 2.0 * T * H * vd * R)
+
+
+def run_minerax(args) -> dict:
+    torch.manual_seed(0)
+    d, H, G, dim, RH, rd, rv, window = 4096, 32, 8, 128, 32, 64, 128, 1024
+    res = {"width": d, "streams": 2, "heads": [H, G], "head": dim, "recurrent_heads": [RH, rd, rv],
+           "latent": [512, 64], "window": window}
+    for name, lens, q_lens, key in (("prefill", [2048, 600], [2048, 600], "prefill_step_rows"),
+                                    ("decode", [600] * 64, [1] * 64, "decode_step_64_rows")):
+        mine, like = {}, {}
+        pre = name == "prefill"
+        rl, sl, first = ([2048, 2048], [0, 63], 0) if pre else ([1] * 64, list(range(64)), 600)
+        T = sum(rl)
+        arows = _runs(q_lens, list(range(len(q_lens))), 0 if pre else 599)
+        _x_rows(T, d, mine)
+        _x_attention(H, G, dim, lens, q_lens, arows, mine, name)
+        _x_latent(H, lens, q_lens, window, mine, name)
+        _b_recurrence(T, RH, rd, rv, _runs(rl, sl, first), mine, not pre)
+        mine.pop("gated_linear_recurrence (gla)")
+        _b_rows(T, d, like)
+        _m_rows(T, d, like)
+        _n_rows(T, d, rl, sl, like, first)
+        _n_attention("window", H, G, lens, q_lens, like, name, 4096, 0)
+        _n_attention("keyval", H, G, lens, q_lens, like, name)
+        _n_attention("latent", H, G, lens, q_lens, like, name, window, 0)
+        for k in [k for k in like if "route" in k]:
+            like.pop(k)
+        res[key] = {"minerax": mine, "like": like, "rows": [T, sum(q_lens)]}
+    return res

@@ -630,6 +630,8 @@ def minerax_from_json(d: dict, name: str | None = None) -> LayeredConfig:
                               float(m["scale"]), kv_rank=int(m["kv_rank"]), rot_dim=int(m["rot_dim"]),
                               window=int((m.get("mask") or {}).get("size", 0)), rot_neighbours=True,
                               out_gate=True, **_rot(m, i, int(m["rot_dim"])))
+            if mixer.rot_dim < 1:
+                raise ValueError(f"layer {i}: rot_dim must be at least 1")
         else:
             raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
         for p in mixer.mixers:

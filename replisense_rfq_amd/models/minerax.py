@@ -166,18 +166,17 @@ class MineraxLM:
         pool = self.kv_k[li]
         pr = ops.matmul_nt(h, lw["proj"])                   # q | dkv | gate
         nq, (g0, gn) = H * (dim + rd), lw["seg"]["g"]
-        qf = torch.empty((T, H, dim + rd), dtype=torch.float32, device=dev)
+        # one (R + rd)-wide fp32 query per head: the plain part carried into the latent space (read
+        # as the projection left it) beside the rotated part
+        q = torch.empty((T, H, R + rd), dtype=torch.float32, device=dev)
+        qn = pr[:, :nq].unflatten(1, (H, dim + rd))[:, :, :dim].transpose(0, 1)
+        ops.bmm_f32(qn, lw["uk"], out=q[:, :, :R].transpose(0, 1))
         ops.qk_norm_rotary_append(pr, None, None, lw["dkv_norm"], False, R, self.cfg.rms_eps,
                                   m.positions[:T], lw["inv_freq"], lw["rot_mult"], dim, R,
-                                  m.slot_mapping[:T], pool, None, H, 1, dim + rd, R + rd, 0, 2, qf,
+                                  m.slot_mapping[:T], pool, None, H, 1, dim + rd, R + rd, 0, 2, q[:, :, R:],
                                   neighbours=mx.rot_neighbours)
-        # the plain query part carried into the latent space (fp32: a score operand) beside the
-        # rotated part: one (R + rd)-wide query per head
-        qn = pr[:, :nq].unflatten(1, (H, dim + rd))[:, :, :dim].transpose(0, 1)
-        qa = ops.bmm_f32(qn, lw["uk"])                                              # [H, T, R]
-        qfull = torch.cat([qa.transpose(0, 1), qf[:, :, dim:]], -1)
         lat = torch.empty((T, H * R), dtype=dt, device=dev)
-        self._attend(m, mx, qfull, pool, pool, R, lw["sink"], lat)
+        self._attend(m, mx, q, pool, pool, R, lw["sink"], lat)
         ov = torch.bmm(lat.view(T, H, R).transpose(0, 1), lw["uv_t"])               # [H, T, vdim]
         y = ops.gate_heads(ov, pr[:, g0:g0 + gn], torch.empty((T, H * vd), dtype=dt, device=dev))
         return ops.matmul_nt(y, lw["o"])

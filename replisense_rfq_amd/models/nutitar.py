@@ -137,19 +137,17 @@ class NutitarLM:
         pr = ops.matmul_nt(hs, lw["proj"])                  # q | dkv | gate  (or q | gate)
         nq = H * (dim + rd)
         gate = pr[:, nq + (R + rd if own else 0):]
-        qf = torch.empty((T, H, dim + rd), dtype=torch.float32, device=dev)
+        # one (R + rd)-wide fp32 query per head: the plain part carried into the latent space (read
+        # as the projection left it) beside the rotated part
+        q = torch.empty((T, H, R + rd), dtype=torch.float32, device=dev)
+        qn = pr[:, :nq].unflatten(1, (H, dim + rd))[:, :, :dim].transpose(0, 1)
+        ops.bmm_f32(qn, lw["uk"], out=q[:, :, :R].transpose(0, 1))
         ops.qk_norm_rotary_append(pr, None, None, lw["dkv_norm"] if own else None, False, R,
                                   self.cfg.rms_eps, m.positions[:T], lw["inv_freq"], lw["rot_mult"],
                                   dim, R, m.slot_mapping[:T], pool if own else None, None, H,
-                                  1 if own else 0, dim + rd, R + rd, 0, 2, qf)
-        # the plain query part (untouched by the kernel above: read as the projection left it)
-        # carried into the latent space, fp32 (a score operand), beside the rotated part: one
-        # (R + rd)-wide query per head
-        qn = pr[:, :nq].unflatten(1, (H, dim + rd))[:, :, :dim].transpose(0, 1)
-        qa = ops.bmm_f32(qn, lw["uk"])                                              # [H, T, R]
-        qfull = torch.cat([qa.transpose(0, 1), qf[:, :, dim:]], -1)
+                                  1 if own else 0, dim + rd, R + rd, 0, 2, q[:, :, R:])
         lat = torch.empty((T, H * R), dtype=dt, device=dev)
-        self._attend(m, qfull, pool, pool, R, lw["sink"], gate, lat, mx)
+        self._attend(m, q, pool, pool, R, lw["sink"], gate, lat, mx)
         ov = torch.bmm(lat.view(T, H, R).transpose(0, 1), lw["uv_t"])               # [H, T, vdim]
         return ops.matmul_nt(ov.transpose(0, 1).reshape(T, H * vd), lw["o"])
 

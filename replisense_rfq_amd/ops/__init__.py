@@ -1142,22 +1142,23 @@ def glu_clamped(gate_up, limit: float, alpha: float = 1.702, out=None):
 _BMM_OUT_DTYPE = None
 
 
-def bmm_f32(a, b):
+def bmm_f32(a, b, out=None):
     """Batched a[B, M, K] . b[B, K, N] on the vendor library with an fp32 result (the
-    accumulator's precision is kept for bf16 operands)."""
+    accumulator's precision is kept for bf16 operands); ``out`` may be a slice of wider rows."""
     if a.dtype == torch.float32:
-        return torch.bmm(a, b)
+        return torch.bmm(a, b) if out is None else torch.bmm(a, b, out=out)
     global _BMM_OUT_DTYPE
     if a.is_cuda and a.shape[1] > 0 and _BMM_OUT_DTYPE is not False:
         if _BMM_OUT_DTYPE:
-            return torch.bmm(a, b, out_dtype=torch.float32)
+            return torch.bmm(a, b, out_dtype=torch.float32, out=out)
         try:                                   # first call (never inside a graph capture)
-            y = torch.bmm(a, b, out_dtype=torch.float32)
+            y = torch.bmm(a, b, out_dtype=torch.float32, out=out)
             _BMM_OUT_DTYPE = True
             return y
         except (TypeError, RuntimeError):
             _BMM_OUT_DTYPE = False
-    return torch.bmm(a.float(), b.float())
+    y = torch.bmm(a.float(), b.float())
+    return y if out is None else out.copy_(y)
 
 
 LATENT_MFMA = os.environ.get("RFQ_LATENT_MFMA", "1") != "0"     # bf16: MFMA tiles where sizes fit

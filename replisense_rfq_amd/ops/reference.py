@@ -782,7 +782,8 @@ def qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all: bool, k_norm
     projection (``norm_all``; weights [H qw], [G kw]) or per head, q over its qw entries
     (weight [qw]) and k over its leading ``k_norm_n`` entries (weight [k_norm_n]); a weight of
     None means no norm.  Then the half-split rotation (``neighbours``: in pairs of neighbouring
-    entries) of entries rot_off .. rot_off + 2 n of every head.  q goes to q_out [T, H, qw] fp32; k rows into k_cache [blocks, G, BS, kw];
+    entries) of entries rot_off .. rot_off + 2 n of every head.  q goes to q_out [T, H, qw] fp32 (or the trailing entries of every head to a
+    narrower q_out); k rows into k_cache [blocks, G, BS, kw];
     values into v_cache [blocks, G, BS, vdim]: v_mode 0 the v columns, 1 the keys as projected
     (before norm and rotation), 2 none.  ``v_out`` [T, G vdim] fp32 receives the values as
     projected; with ``v_in`` [T, G vdim] fp32 the cached ones are (1 - v_take) v + v_take v_in.
@@ -815,7 +816,7 @@ def qk_norm_rotary_append(proj, bias, q_norm_w, k_norm_w, norm_all: bool, k_norm
             k[..., :k_norm_n] = _rms(k[..., :k_norm_n], eps) * k_norm_w.float()
     q = _rotate_halves(q, positions[:T], inv_freq, rot_mult, q_rot_off, neighbours)
     k = _rotate_halves(k, positions[:T], inv_freq, rot_mult, k_rot_off, neighbours)
-    q_out.copy_(q)
+    q_out.copy_(q[..., qw - q_out.shape[2]:])
     if k_cache is None or G == 0:
         return
     v = x[:, nq + nk:nq + nk + G * vdim].reshape(T, G, vdim) if v_mode == 0 else raw_k

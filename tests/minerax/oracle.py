@@ -229,3 +229,10 @@ def forward(cfg, tensors, tokens, layers=None):
         if layers is not None:
             layers.append(x.sum(0))
     return layer_norm(x.sum(0), w["final.norm"], eps) @ w["head"].T * cfg["logit_scale"]
+
+
+def greedy(cfg, tensors, prompt, n):
+    toks = list(prompt)
+    for _ in range(n):
+        toks.append(int(forward(cfg, tensors, toks)[-1].argmax()))
+    return toks[len(prompt):]
