@@ -231,113 +231,199 @@ __global__ __launch_bounds__(256) void linrec_finish_kernel(
 }
 
 // The scan of a long step: decays formed ahead (z holds them), read-outs to `raw` for the
-// row-parallel norm and gate.  One WAVE per (run, head, 64 value channels), no LDS and no
-// barrier: every wave loads the token's q, k and decay itself, a key channel per lane (two for
-// dim 128), and broadcasts channel i to all lanes with v_readlane, so the sums run on scalar
-// operands; the next token's operands are loaded while the current one is summed.
+// row-parallel norm and gate.  One workgroup of four waves per (run, head, 64 value channels).  Four
+// neighbouring lanes share a value channel: each holds a quarter of the key channels of its column
+// of S in registers, and the sums over all of them finish with two DPP adds inside the quad.  The
+// operands of SCAN_ROWS tokens at a time pass through LDS (a lane reads its key channels in 16-byte
+// pieces, one address per quarter); the next tokens' are in flight meanwhile.
+// NR = 32, 64 or 128 key channels, of which `dim` exist (the others are zeros throughout).
+// LDS (floats): SCAN_ROWS x (decay[NR] | k[NR] | q[NR] | v[64]) | beta[SCAN_ROWS]
+namespace {
+constexpr int SCAN_ROWS = 16;
+
+__device__ __forceinline__ float quad_sum(float v) {
+  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xf, 0xf, true));   // lanes 1 0 3 2
+  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x4E, 0xf, 0xf, true));   // lanes 2 3 0 1
+  return v;
+}
+
+// entries c .. c + 3 of a row of n; entries past its end are zeros
+__device__ __forceinline__ float4 row4(const float* p, int c, int n, bool vec) {
+  if (vec && c + 3 < n) return *reinterpret_cast<const float4*>(p + c);
+  return make_float4(c < n ? p[c] : 0.f, c + 1 < n ? p[c + 1] : 0.f, c + 2 < n ? p[c + 2] : 0.f,
+                     c + 3 < n ? p[c + 3] : 0.f);
+}
+__device__ __forceinline__ float4 row4(const bf16_t* p, int c, int n, bool vec) {
+  if (vec && c + 3 < n) {
+    const uint2 w = *reinterpret_cast<const uint2*>(p + c);
+    return make_float4(__uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u),
+                       __uint_as_float(w.y << 16), __uint_as_float(w.y & 0xffff0000u));
+  }
+  return make_float4(c < n ? ldf(p + c) : 0.f, c + 1 < n ? ldf(p + c + 1) : 0.f,
+                     c + 2 < n ? ldf(p + c + 2) : 0.f, c + 3 < n ? ldf(p + c + 3) : 0.f);
+}
+}  // namespace
+
 template <typename TI, typename TG, int NR, bool DELTA>
-__global__ __launch_bounds__(64) void gated_linrec_scan_kernel(
+__global__ __launch_bounds__(256) void gated_linrec_scan_kernel(
     const TI* __restrict__ q, const TI* __restrict__ k, const TI* __restrict__ v,
     int64_t q_stride, int64_t k_stride, int64_t v_stride, const float* __restrict__ z,
     int64_t z_stride, const TG* __restrict__ beta, int64_t b_stride, float q_scale,
     float* __restrict__ raw, float* __restrict__ state, const int32_t* __restrict__ row_state,
     const int32_t* __restrict__ row_back, const int32_t* __restrict__ row_fwd,
-    const int32_t* __restrict__ pos, const int32_t* __restrict__ run_rows, int H, int rep,
-    int vdim, int slots) {
-  constexpr int dim = NR, C = (NR + 63) / 64;
+    const int32_t* __restrict__ pos, const int32_t* __restrict__ run_rows, int H, int rep, int dim,
+    int vdim, int slots, int vec) {
+  constexpr int NK = NR / 4;                           // key channels per lane
+  constexpr int P4 = NR / 4;                           // 16-byte pieces per row of q, k, decay
+  constexpr int NL = (SCAN_ROWS * P4 + 255) / 256;     // pieces per thread
+  constexpr int RS = 3 * NR + 64;                      // floats per token in LDS
   const int t0 = run_rows != nullptr ? run_rows[blockIdx.x] : (int)blockIdx.x;
   const int h = blockIdx.y;
   if (t0 < 0 || row_back[t0] != 0) return;
   const int n = row_fwd[t0] + 1;
   const int code = row_state[t0];
-  const int lane = threadIdx.x;
-  const int j = blockIdx.z * 64 + lane;                // this lane's value channel
+  const int tid = threadIdx.x, lane = tid & 63, ks = lane & 3;
+  const int v0 = blockIdx.z * 64;
+  const int jl = (tid >> 6) * 16 + (lane >> 2);        // value channel inside the workgroup
+  const int j = v0 + jl;
   const bool vlive = j < vdim;
   const int hq = h / rep;
-  const int vc = h * vdim + (vlive ? j : 0);
+  const int nv = min(64, vdim - v0);
 
-  float sreg[NR];
+  __shared__ __attribute__((aligned(16))) float ops[SCAN_ROWS * RS];
+  __shared__ float bet[SCAN_ROWS];
+
+  float sreg[NK];
   const bool from_state = code >= 0 && pos[t0] > 0;
   const int64_t hsz = (int64_t)dim * vdim;
   const float* rd = state + (((int64_t)(code & 1) * slots + (code >> 1)) * H + h) * hsz;
 #pragma unroll
-  for (int i = 0; i < NR; ++i) sreg[i] = (from_state && vlive) ? rd[i * vdim + j] : 0.f;
+  for (int i = 0; i < NK; ++i) {
+    const int ch = ks * NK + i;
+    sreg[i] = (from_state && vlive && ch < dim) ? rd[(int64_t)ch * vdim + j] : 0.f;
+  }
 
-  float nq[C], nk[C], na[C], nv = 0.f, nb = 0.f;
-  auto load = [&](int64_t t) {
+  float4 rq[NL], rk[NL], ra[NL], rv;
+  float rb = 0.f;
+  auto fetch = [&](int a0) {
+    const int rows = min(SCAN_ROWS, n - a0);
 #pragma unroll
-    for (int c = 0; c < C; ++c) {
-      const int ch = c * 64 + lane;
-      const bool ok = ch < dim;
-      nq[c] = ok ? ldf(q + t * q_stride + hq * dim + ch) : 0.f;
-      nk[c] = ok ? ldf(k + t * k_stride + hq * dim + ch) : 0.f;
-      na[c] = ok ? z[t * z_stride + h * dim + ch] : 0.f;
+    for (int u = 0; u < NL; ++u) {
+      const int x = tid + u * 256, r = x / P4, c = (x - r * P4) * 4;
+      if (x < SCAN_ROWS * P4 && r < rows) {
+        const int64_t t = t0 + a0 + r;
+        rq[u] = row4(q + t * q_stride + (int64_t)hq * dim, c, dim, vec);
+        rk[u] = row4(k + t * k_stride + (int64_t)hq * dim, c, dim, vec);
+        ra[u] = row4(z + t * z_stride + (int64_t)h * dim, c, dim, vec);
+      }
     }
-    if (vlive) nv = ldf(v + t * v_stride + vc);
-    if (DELTA) nb = ldf(beta + t * b_stride + h);
+    {
+      const int r = tid >> 4, c = (tid & 15) * 4;      // 16 rows x 16 pieces of 64 value channels
+      if (r < rows) rv = row4(v + (t0 + a0 + r) * v_stride + (int64_t)h * vdim + v0, c, nv, vec);
+    }
+    if (DELTA && tid < rows) rb = ldf(beta + (int64_t)(t0 + a0 + tid) * b_stride + h);
   };
-  load(t0);
-  for (int a = 0; a < n; ++a) {
-    int cq[C], ck[C], ca[C];
+  fetch(0);
+  for (int a0 = 0; a0 < n; a0 += SCAN_ROWS) {
+    const int rows = min(SCAN_ROWS, n - a0);
+    __syncthreads();                                   // the last tokens' reads are done
 #pragma unroll
-    for (int c = 0; c < C; ++c) {
-      cq[c] = __float_as_int(nq[c]);
-      ck[c] = __float_as_int(nk[c]);
-      ca[c] = __float_as_int(na[c]);
-    }
-    const float vj = nv;
-    const float bj = DELTA ? 1.0f / (1.0f + expf(-nb)) : 1.f;
-    if (a + 1 < n) load(t0 + a + 1);
-    float po[4] = {0.f, 0.f, 0.f, 0.f};
-    if (DELTA) {
-      float pa[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int i = 0; i < NR; ++i) {
-        const float ai = __int_as_float(__builtin_amdgcn_readlane(ca[i >> 6], i & 63));
-        const float ki = __int_as_float(__builtin_amdgcn_readlane(ck[i >> 6], i & 63));
-        sreg[i] *= ai;
-        pa[i & 3] += sreg[i] * ki;
-      }
-      const float u = bj * (vj - ((pa[0] + pa[1]) + (pa[2] + pa[3])));
-#pragma unroll
-      for (int i = 0; i < NR; ++i) {
-        const float ki = __int_as_float(__builtin_amdgcn_readlane(ck[i >> 6], i & 63));
-        const float qi = __int_as_float(__builtin_amdgcn_readlane(cq[i >> 6], i & 63));
-        sreg[i] += ki * u;
-        po[i & 3] += sreg[i] * qi;
-      }
-    } else {
-#pragma unroll
-      for (int i = 0; i < NR; ++i) {
-        const float ai = __int_as_float(__builtin_amdgcn_readlane(ca[i >> 6], i & 63));
-        const float ki = __int_as_float(__builtin_amdgcn_readlane(ck[i >> 6], i & 63));
-        const float qi = __int_as_float(__builtin_amdgcn_readlane(cq[i >> 6], i & 63));
-        sreg[i] = ai * sreg[i] + ki * vj;
-        po[i & 3] += sreg[i] * qi;
+    for (int u = 0; u < NL; ++u) {
+      const int x = tid + u * 256, r = x / P4, c = (x - r * P4) * 4;
+      if (x < SCAN_ROWS * P4 && r < rows) {
+        float* o = ops + r * RS + c;
+        *reinterpret_cast<float4*>(o) = ra[u];
+        *reinterpret_cast<float4*>(o + NR) = rk[u];
+        *reinterpret_cast<float4*>(o + 2 * NR) = rq[u];
       }
     }
-    if (vlive) raw[(int64_t)(t0 + a) * H * vdim + vc] = ((po[0] + po[1]) + (po[2] + po[3])) * q_scale;
+    if ((tid >> 4) < rows) *reinterpret_cast<float4*>(ops + (tid >> 4) * RS + 3 * NR + (tid & 15) * 4) = rv;
+    if (DELTA && tid < rows) bet[tid] = 1.0f / (1.0f + expf(-rb));
+    __syncthreads();
+    if (a0 + SCAN_ROWS < n) fetch(a0 + SCAN_ROWS);     // in flight during the sums
+    float4 ca[NK / 4], ck[NK / 4], cq[NK / 4];         // a token's operands, read one token ahead
+    float cv, cb = 1.f;
+    auto operands = [&](int r) {
+      const float* row = ops + r * RS + ks * NK;
+#pragma unroll
+      for (int i = 0; i < NK / 4; ++i) {
+        ca[i] = *reinterpret_cast<const float4*>(row + 4 * i);
+        ck[i] = *reinterpret_cast<const float4*>(row + NR + 4 * i);
+        cq[i] = *reinterpret_cast<const float4*>(row + 2 * NR + 4 * i);
+      }
+      cv = ops[r * RS + 3 * NR + jl];
+      if (DELTA) cb = bet[r];
+    };
+    operands(0);
+#pragma unroll 2
+    for (int r = 0; r < rows; ++r) {
+      float4 da[NK / 4], dk[NK / 4], dq[NK / 4];
+#pragma unroll
+      for (int i = 0; i < NK / 4; ++i) {
+        da[i] = ca[i];
+        dk[i] = ck[i];
+        dq[i] = cq[i];
+      }
+      const float vj = cv, bj = cb;
+      operands(r + 1 < rows ? r + 1 : r);
+      float po[4] = {0.f, 0.f, 0.f, 0.f};
+      if (DELTA) {
+        float pa[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < NK / 4; ++i) {
+          pa[0] += (sreg[4 * i] *= da[i].x) * dk[i].x;
+          pa[1] += (sreg[4 * i + 1] *= da[i].y) * dk[i].y;
+          pa[2] += (sreg[4 * i + 2] *= da[i].z) * dk[i].z;
+          pa[3] += (sreg[4 * i + 3] *= da[i].w) * dk[i].w;
+        }
+        const float u = bj * (vj - quad_sum((pa[0] + pa[1]) + (pa[2] + pa[3])));
+#pragma unroll
+        for (int i = 0; i < NK / 4; ++i) {
+          po[0] += (sreg[4 * i] += dk[i].x * u) * dq[i].x;
+          po[1] += (sreg[4 * i + 1] += dk[i].y * u) * dq[i].y;
+          po[2] += (sreg[4 * i + 2] += dk[i].z * u) * dq[i].z;
+          po[3] += (sreg[4 * i + 3] += dk[i].w * u) * dq[i].w;
+        }
+      } else {
+#pragma unroll
+        for (int i = 0; i < NK / 4; ++i) {
+          po[0] += (sreg[4 * i] = da[i].x * sreg[4 * i] + dk[i].x * vj) * dq[i].x;
+          po[1] += (sreg[4 * i + 1] = da[i].y * sreg[4 * i + 1] + dk[i].y * vj) * dq[i].y;
+          po[2] += (sreg[4 * i + 2] = da[i].z * sreg[4 * i + 2] + dk[i].z * vj) * dq[i].z;
+          po[3] += (sreg[4 * i + 3] = da[i].w * sreg[4 * i + 3] + dk[i].w * vj) * dq[i].w;
+        }
+      }
+      const float o = quad_sum((po[0] + po[1]) + (po[2] + po[3])) * q_scale;
+      if (ks == 0 && vlive) raw[(int64_t)(t0 + a0 + r) * H * vdim + (int64_t)h * vdim + j] = o;
+    }
   }
   if (code >= 0 && vlive) {
     float* wr = state + (((int64_t)(1 - (code & 1)) * slots + (code >> 1)) * H + h) * hsz;
 #pragma unroll
-    for (int i = 0; i < NR; ++i) wr[i * vdim + j] = sreg[i];
+    for (int i = 0; i < NK; ++i) {
+      const int ch = ks * NK + i;
+      if (ch < dim) wr[(int64_t)ch * vdim + j] = sreg[i];
+    }
   }
 }
 
 // ------------------------------------------------------------------ launchers
 template <typename TI, typename TG, int NR, bool DELTA>
+static void launch_linrec_scan(const LinrecArgs& a, hipStream_t s) {
+  auto al = [](const void* p, int64_t stride, int64_t head, size_t esz) {
+    return reinterpret_cast<uintptr_t>(p) % (4 * esz) == 0 && stride % 4 == 0 && head % 4 == 0;
+  };
+  const bool vec = al(a.q, a.qs, a.dim, sizeof(TI)) && al(a.k, a.ks, a.dim, sizeof(TI)) &&
+                   al(a.v, a.vs, a.vdim, sizeof(TI)) && al(a.z, a.zs, a.dim, 4);
+  const dim3 grid(a.run_rows != nullptr ? a.runs : a.T, a.H, (a.vdim + 63) / 64);
+  hipLaunchKernelGGL((gated_linrec_scan_kernel<TI, TG, NR, DELTA>), grid, dim3(256), 0, s,
+                     (const TI*)a.q, (const TI*)a.k, (const TI*)a.v, a.qs, a.ks, a.vs, a.z, a.zs,
+                     (const TG*)a.beta, a.bs, a.q_scale, a.raw, a.state, a.row_state, a.row_back,
+                     a.row_fwd, a.pos, a.run_rows, a.H, a.rep, a.dim, a.vdim, a.slots, (int)vec);
+}
+
+template <typename TI, typename TG, int NR, bool DELTA>
 static void launch_linrec_one(const LinrecArgs& a, hipStream_t s) {
-  if constexpr (NR > 0) {
-    if (a.raw != nullptr && a.decay_ready) {
-      const dim3 grid(a.run_rows != nullptr ? a.runs : a.T, a.H, (a.vdim + 63) / 64);
-      hipLaunchKernelGGL((gated_linrec_scan_kernel<TI, TG, NR, DELTA>), grid, dim3(64), 0, s,
-                         (const TI*)a.q, (const TI*)a.k, (const TI*)a.v, a.qs, a.ks, a.vs, a.z, a.zs,
-                         (const TG*)a.beta, a.bs, a.q_scale, a.raw, a.state, a.row_state,
-                         a.row_back, a.row_fwd, a.pos, a.run_rows, a.H, a.rep, a.vdim, a.slots);
-      return;
-    }
-  }
   const int threads = ((a.dim > a.vdim ? a.dim : a.vdim) + 63) / 64 * 64;
   const size_t lds = (size_t)(8 * a.dim + 16 + (NR > 0 ? 0 : a.dim * a.vdim)) * 4;
   static bool attr = false;
@@ -357,6 +443,12 @@ static void launch_linrec_one(const LinrecArgs& a, hipStream_t s) {
 
 template <typename TI, typename TG, bool DELTA>
 static void launch_linrec_dim(const LinrecArgs& a, hipStream_t s) {
+  if (a.raw != nullptr && a.decay_ready && a.dim <= 128) {
+    if (a.dim <= 32) launch_linrec_scan<TI, TG, 32, DELTA>(a, s);
+    else if (a.dim <= 64) launch_linrec_scan<TI, TG, 64, DELTA>(a, s);
+    else launch_linrec_scan<TI, TG, 128, DELTA>(a, s);
+    return;
+  }
   if (a.dim == 32) launch_linrec_one<TI, TG, 32, DELTA>(a, s);
   else if (a.dim == 64) launch_linrec_one<TI, TG, 64, DELTA>(a, s);
   else if (a.dim == 128) launch_linrec_one<TI, TG, 128, DELTA>(a, s);
