@@ -1,6 +1,6 @@
 // Row kernels of layers around several residual streams:
 //
-//   streams_norm    x_t <- sum_s mix[s, t] x_s + w_out[t] y (all streams from the old ones), then
+//   streams_norm    x_t <- sum_s mix[s, t] x_s + w_out[t] y (the previous streams on the right),
 //                   u = sum_s w_in[s] x_s and out = norm(u) w for the next sublayer (layer norm
 //                   without bias, or RMS norm): one kernel per sublayer boundary.  The first one
 //                   starts the streams from the embedding table, the last one need not write them.

@@ -7,7 +7,7 @@ Every row holds S residual streams x_1 .. x_S (fp32):
   x_s = embed[token] for all s
   per sublayer (mixer, feed-forward):
     u = sum_s in[s] x_s;  y = sublayer(layer_norm(u) w)
-    x_t <- sum_s mix[s, t] x_s + out[t] y        all streams from the old ones
+    x_t <- sum_s mix[s, t] x_s + out[t] y        with the previous streams on the right
   logits = head . (layer_norm(sum_s x_s) w_final) * logit_scale
 
 The update of the streams, the next sublayer's weighted sum and its norm are one kernel

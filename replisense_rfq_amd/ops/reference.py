@@ -981,8 +981,8 @@ def mlstm_recurrence(q, k, v, z, zbias, cap: float, q_scale: float, gate, norm_w
 # Several residual streams, a gated tanh-gelu unit, gated heads.
 def streams_norm(x, y, mix, w_out, w_in, w, eps: float, centre: bool, out, keep: bool, ids, table) -> None:
     """x [T, S, d] fp32 holds S residual streams of every row.  With ``ids`` they all start as the
-    rows of ``table``.  With ``y`` [T, d]: x_t <- sum_s mix[s, t] x_s + w_out[t] y, all streams from
-    the old ones.  u = sum_s w_in[s] x_s; out = w u / sqrt(mean(u^2) + eps), ``centre``: with
+    rows of ``table``.  With ``y`` [T, d]: x_t <- sum_s mix[s, t] x_s + w_out[t] y, the previous
+    streams on the right.  u = sum_s w_in[s] x_s; out = w u / sqrt(mean(u^2) + eps), ``centre``: with
     u less its mean (a layer norm without bias).  ``keep`` False: x need not be written (nobody
     reads it afterwards)."""
     if ids is not None:

@@ -52,7 +52,8 @@ def streams_in(streams, w_in):
 
 
 def streams_update(streams, mix, w_out, y):
-    """All streams at once from the old ones: x_t <- sum_s mix[s, t] x_s + out[t] y."""
+    """Every new stream t is a mixture of the previous streams plus its share of y; row s of mix holds
+    what stream s gives."""
     S = streams.shape[0]
     return torch.stack([sum(float(mix[s, t]) * streams[s] for s in range(S)) + float(w_out[t]) * y
                         for t in range(S)])

@@ -40,8 +40,8 @@ def run_rows(cuts, slot):
 @pytest.mark.parametrize("S", [1, 2, 3, 4, 5, 8])
 @pytest.mark.parametrize("d", [37, 44, 256, 2052])
 def test_streams_update_weighted_sum_and_norm(device, S, d):
-    """All streams move at once from the old ones, mix is indexed [from, to]; the next sublayer
-    reads the layer norm of a weighted sum."""
+    """Every new stream is formed from the previous ones (row s of mix: what stream s gives); the
+    next sublayer reads the layer norm of a weighted sum."""
     g = torch.Generator().manual_seed(1)
     T, eps = 5, 1e-3
     x = torch.randn(T, S, d, generator=g) * 3 + 1.5

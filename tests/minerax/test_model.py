@@ -271,6 +271,40 @@ def test_checkpoint_folder_round_trip(device, tmp_path):
     check(run_schedule(eng, alone(t, [9, 2])), cfg, full, {"a": t})
 
 
+def test_trace_replay_from_the_command_line(tmp_path):
+    """bin/trace_run chooses the model by the folder's config.json and writes the wanted logits."""
+    import json
+    import os
+    import subprocess
+
+    import numpy as np
+    from safetensors.torch import save_file
+
+    cfg = SMALL
+    _, full = build(cfg, "cpu")
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    save_file({k: v.to(torch.bfloat16).contiguous() for k, v in full.items()},
+              str(tmp_path / "model.safetensors"))
+    a, b = tokens(60, cfg["vocab"], 1), tokens(9, cfg["vocab"], 2)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:40], "want": [0, 39]},
+                                     {"id": "b", "tokens": b[:2], "want": []}], "end": []},
+             {"step": 1, "entries": [{"id": "b", "tokens": b[2:], "want": [6]},
+                                     {"id": "a", "tokens": a[40:], "want": [19]}], "end": ["a", "b"]},
+             {"step": 2, "entries": [{"id": "a", "tokens": b, "want": [8]}], "end": ["a"]}]    # name reused
+    out = tmp_path / "out"
+    root = os.path.dirname(os.path.dirname(os.path.dirname(os.path.abspath(__file__))))
+    p = subprocess.run([os.path.join(root, "bin", "trace_run"), "--model", str(tmp_path), "--dtype", "float32",
+                        "--out", str(out), "--max-tokens", "128", "--device", "cpu"],
+                       input="\n".join(json.dumps(s) for s in steps) + "\n", text=True,
+                       capture_output=True, timeout=300)
+    assert p.returncode == 0, p.stderr[-2000:]
+    ra, rb = oracle.forward(cfg, full, a), oracle.forward(cfg, full, b)
+    for n, rows in {0: [ra[0], ra[39]], 1: [rb[8], ra[59]], 2: [rb[8]]}.items():
+        got = np.fromfile(out / f"{n}.f32", dtype="<f4").reshape(len(rows), cfg["vocab"])
+        for g, r in zip(got, rows):
+            assert float(np.abs(g - r.numpy()).max() / r.abs().max()) < 3e-4
+
+
 def test_named_configuration_and_registry():
     from replisense_rfq_amd.models import layered_model_class
     from replisense_rfq_amd.models.config import get_config
